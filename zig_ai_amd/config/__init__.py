@@ -19,6 +19,7 @@ from .rudilix import RudilixConfig  # noqa: F401
 from .ranesun import RanesunConfig  # noqa: F401
 from .gemodra import GemodraConfig  # noqa: F401
 from .nopozen import NopozenConfig  # noqa: F401
+from .vupelorn import VupelornConfig  # noqa: F401
 
 _ARCHITECTURES: Dict[str, Any] = {}
 
@@ -72,3 +73,4 @@ register_architecture("Rudilix", RudilixConfig)
 register_architecture("Ranesun", RanesunConfig)
 register_architecture("Gemodra", GemodraConfig)
 register_architecture("Nopozen", NopozenConfig)
+register_architecture("Vupelorn", VupelornConfig)

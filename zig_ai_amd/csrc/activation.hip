@@ -124,17 +124,23 @@ extern "C" int za_copy_columns(const void* in, int in_dtype, int in_width, int c
 // A gated linear unit with bounded inputs, on the fused gate|up projection:
 //   g = min(gu[t, i], limit);  u = clamp(gu[t, I + i], -limit, limit)
 //   out[t, i] = g * sigmoid(alpha * g) * (u + up_offset)
-// in 32-bit.  `limit <= 0` means no bound.
+// in 32-bit.  `limit <= 0` means no bound.  With `row_scale` (one number a row) both inputs
+// are multiplied by it first: what a linear projection gives for an input so scaled.
 template <typename T>
 __global__ void __launch_bounds__(256)
-clamped_glu_kernel(const T* __restrict__ gu, T* __restrict__ out, int n_tokens, int inter,
-                   float limit, float alpha, float up_offset) {
+clamped_glu_kernel(const T* __restrict__ gu, T* __restrict__ out,
+                   const float* __restrict__ row_scale, int n_tokens, int inter, float limit,
+                   float alpha, float up_offset) {
   const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   const size_t total = (size_t)n_tokens * inter;
   if (idx >= total) return;
   const size_t t = idx / inter, i = idx % inter;
   float g = to_f32<T>(gu[t * 2 * inter + i]);
   float u = to_f32<T>(gu[t * 2 * inter + inter + i]);
+  if (row_scale) {
+    g *= row_scale[t];
+    u *= row_scale[t];
+  }
   if (limit > 0.f) {
     g = fminf(g, limit);
     u = fminf(fmaxf(u, -limit), limit);
@@ -144,8 +150,9 @@ clamped_glu_kernel(const T* __restrict__ gu, T* __restrict__ out, int n_tokens, 
 
 template <typename T>
 __global__ void __launch_bounds__(256)
-clamped_glu_vec8_kernel(const T* __restrict__ gu, T* __restrict__ out, int n_tokens, int inter,
-                        float limit, float alpha, float up_offset) {
+clamped_glu_vec8_kernel(const T* __restrict__ gu, T* __restrict__ out,
+                        const float* __restrict__ row_scale, int n_tokens, int inter, float limit,
+                        float alpha, float up_offset) {
   const size_t idx = ((size_t)blockIdx.x * blockDim.x + threadIdx.x) * 8;
   const size_t total = (size_t)n_tokens * inter;
   if (idx >= total) return;
@@ -153,9 +160,10 @@ clamped_glu_vec8_kernel(const T* __restrict__ gu, T* __restrict__ out, int n_tok
   float g[8], u[8], o[8];
   load8<T>(gu + t * 2 * inter + i, g);
   load8<T>(gu + t * 2 * inter + inter + i, u);
+  const float rs = row_scale ? row_scale[t] : 1.f;
 #pragma unroll
   for (int k = 0; k < 8; ++k) {
-    float gk = g[k], uk = u[k];
+    float gk = g[k] * rs, uk = u[k] * rs;
     if (limit > 0.f) {
       gk = fminf(gk, limit);
       uk = fminf(fmaxf(uk, -limit), limit);
@@ -165,8 +173,9 @@ clamped_glu_vec8_kernel(const T* __restrict__ gu, T* __restrict__ out, int n_tok
   store8<T>(out + idx, o);
 }
 
-extern "C" int za_clamped_glu(const void* gu, void* out, int dtype, int n_tokens, int inter,
-                              float limit, float alpha, float up_offset, hipStream_t stream) {
+extern "C" int za_clamped_glu(const void* gu, void* out, int dtype, const float* row_scale,
+                              int n_tokens, int inter, float limit, float alpha, float up_offset,
+                              hipStream_t stream) {
   if (n_tokens == 0) return 0;
   if (n_tokens < 0 || inter <= 0 || !gu || !out) return ZA_ERR_ARG;
   const size_t total = (size_t)n_tokens * inter;
@@ -174,8 +183,8 @@ extern "C" int za_clamped_glu(const void* gu, void* out, int dtype, int n_tokens
   const size_t threads = vec ? total / 8 : total;
   dim3 grid((unsigned)((threads + 255) / 256)), block(256);
 #define ZA_GLU(KERNEL, T)                                                                      \
-  hipLaunchKernelGGL((KERNEL<T>), grid, block, 0, stream, (const T*)gu, (T*)out, n_tokens, inter, \
-                     limit, alpha, up_offset)
+  hipLaunchKernelGGL((KERNEL<T>), grid, block, 0, stream, (const T*)gu, (T*)out, row_scale,       \
+                     n_tokens, inter, limit, alpha, up_offset)
   if (dtype == 0) {
     if (vec) ZA_GLU(clamped_glu_vec8_kernel, float); else ZA_GLU(clamped_glu_kernel, float);
   } else if (dtype == 1) {

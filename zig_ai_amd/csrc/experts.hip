@@ -529,12 +529,14 @@ extern "C" int za_route_topk(const float* z, int ld, const float* correction, in
 // An output beyond the n_real experts that have weights hands the token's input x[t] on.
 // gate(t) = sigmoid(gate_logits[t * gate_ld]) when gate_logits is given, else 1; `shared`
 // may be absent.  The sum is taken in the order j = 0 .. top - 1, then the shared expert.
+// `weigh` 0: the experts' outputs hold their weights already (a weight on an expert's input).
 template <typename TE, typename TX>
 __global__ void __launch_bounds__(256)
 experts_combine_kernel(const TE* __restrict__ expert_out, const int* __restrict__ chosen,
                        const float* __restrict__ weight, const TX* __restrict__ x,
                        const TE* __restrict__ shared, const float* __restrict__ gate_logits,
-                       int gate_ld, float* __restrict__ y, int top, int n_real, int width) {
+                       int gate_ld, float* __restrict__ y, int top, int n_real, int width,
+                       int weigh) {
   const size_t t = blockIdx.x;
   float g = 1.0f;
   if (shared && gate_logits) g = 1.0f / (1.0f + expf(-gate_logits[t * gate_ld]));
@@ -542,7 +544,7 @@ experts_combine_kernel(const TE* __restrict__ expert_out, const int* __restrict_
     float acc = 0.f;
     for (int j = 0; j < top; ++j) {
       const int e = chosen[t * top + j];
-      const float w = weight[t * top + j];
+      const float w = (weigh || e >= n_real) ? weight[t * top + j] : 1.f;
       const float v = e < n_real ? to_f32<TE>(expert_out[(t * top + j) * width + i])
                                  : to_f32<TX>(x[t * width + i]);
       acc = fmaf(w, v, acc);
@@ -557,7 +559,7 @@ extern "C" int za_experts_combine(const void* expert_out, int out_dtype, const i
                                   const float* weight, const void* x, int x_dtype,
                                   const void* shared, const float* gate_logits, int gate_ld,
                                   float* y, int n_tokens, int top, int n_real, int width,
-                                  hipStream_t stream) {
+                                  int weigh, hipStream_t stream) {
   if (n_tokens == 0) return 0;
   if (n_tokens < 0 || top <= 0 || width <= 0 || n_real < 0 || !chosen || !weight || !x || !y ||
       (n_real > 0 && !expert_out))
@@ -566,7 +568,7 @@ extern "C" int za_experts_combine(const void* expert_out, int out_dtype, const i
 #define ZA_EC(TE, TX)                                                                          \
   hipLaunchKernelGGL((experts_combine_kernel<TE, TX>), grid, block, 0, stream,                 \
                      (const TE*)expert_out, chosen, weight, (const TX*)x, (const TE*)shared,   \
-                     gate_logits, gate_ld, y, top, n_real, width)
+                     gate_logits, gate_ld, y, top, n_real, width, weigh)
   if (out_dtype == 0 && x_dtype == 0) ZA_EC(float, float);
   else if (out_dtype == 0 && x_dtype == 1) ZA_EC(float, bf16_t);
   else if (out_dtype == 1 && x_dtype == 1) ZA_EC(bf16_t, bf16_t);

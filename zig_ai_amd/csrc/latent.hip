@@ -23,7 +23,7 @@
 //                      of 16 rows each for prompt portions and mixed steps
 //   latent_decode_mfma      steps that only decode: four waves share 16 rows
 // Rotation: adjacent pairs (2i, 2i + 1) or halves (i, i + dims/2) of the first `rot_dims`
-// elements, angle = position * inv_freq[i] in 32-bit.
+// elements, angle = position * inv_freq[i] in 32-bit, cosine and sine times `magnitude`.
 #include <math.h>
 
 #include "common.h"
@@ -38,7 +38,7 @@ latent_prepare_kernel(const T* __restrict__ down, int ld, int q_col, int Rq, int
                       int Dr, const float* __restrict__ q_norm_w, const float* __restrict__ c_norm_w,
                       float eps, const int* __restrict__ positions, const int* __restrict__ slots,
                       const float* __restrict__ inv_freq, int rot_dims, int adjacent,
-                      T* __restrict__ cq, T* __restrict__ plane, int page_size,
+                      float magnitude, T* __restrict__ cq, T* __restrict__ plane, int page_size,
                       long long page_stride) {
   __shared__ float scratch[16];
   const size_t t = blockIdx.x;
@@ -75,6 +75,8 @@ latent_prepare_kernel(const T* __restrict__ down, int ld, int q_col, int Rq, int
     const int a = adjacent ? 2 * i : i, b = adjacent ? 2 * i + 1 : i + half;
     float sn, cs;
     sincosf(pos * inv_freq[i], &sn, &cs);
+    sn *= magnitude;
+    cs *= magnitude;
     const float u = to_f32<T>(kr[a]), v = to_f32<T>(kr[b]);
     dst[R + a] = from_f32<T>(u * cs - v * sn);
     dst[R + b] = from_f32<T>(v * cs + u * sn);
@@ -86,11 +88,12 @@ extern "C" int za_latent_prepare(const void* down, int dtype, int ld, int q_col,
                                  int c_col, int kv_rank, int rot_dim, const float* q_norm_w,
                                  const float* c_norm_w, float eps, const int* positions,
                                  const int* slots, const float* inv_freq, int rot_dims,
-                                 int adjacent, void* cq, void* plane, int page_size,
+                                 int adjacent, float magnitude, void* cq, void* plane, int page_size,
                                  long long page_stride, int n_tokens, hipStream_t stream) {
   if (n_tokens == 0) return 0;
   if (n_tokens < 0 || !down || ld <= 0 || kv_rank <= 0 || rot_dim < 0 || rot_dims < 0 ||
-      rot_dims > rot_dim || rot_dims % 2 != 0 || c_col < 0 || c_col + kv_rank + rot_dim > ld ||
+      rot_dims > rot_dim || rot_dims % 2 != 0 || c_col < 0 ||
+      (plane && c_col + kv_rank + rot_dim > ld) ||
       (cq && (q_rank <= 0 || q_col < 0 || q_col + q_rank > ld || !q_norm_w)) ||
       (plane && (!slots || !c_norm_w || page_size <= 0 || page_stride < (long long)page_size * (kv_rank + rot_dim))) ||
       (plane && rot_dims > 0 && (!inv_freq || !positions)))
@@ -99,12 +102,12 @@ extern "C" int za_latent_prepare(const void* down, int dtype, int ld, int q_col,
   if (dtype == 0)
     hipLaunchKernelGGL((latent_prepare_kernel<float>), grid, block, 0, stream, (const float*)down,
                        ld, q_col, q_rank, c_col, kv_rank, rot_dim, q_norm_w, c_norm_w, eps,
-                       positions, slots, inv_freq, rot_dims, adjacent, (float*)cq, (float*)plane,
+                       positions, slots, inv_freq, rot_dims, adjacent, magnitude, (float*)cq, (float*)plane,
                        page_size, page_stride);
   else if (dtype == 1)
     hipLaunchKernelGGL((latent_prepare_kernel<bf16_t>), grid, block, 0, stream,
                        (const bf16_t*)down, ld, q_col, q_rank, c_col, kv_rank, rot_dim, q_norm_w,
-                       c_norm_w, eps, positions, slots, inv_freq, rot_dims, adjacent, (bf16_t*)cq,
+                       c_norm_w, eps, positions, slots, inv_freq, rot_dims, adjacent, magnitude, (bf16_t*)cq,
                        (bf16_t*)plane, page_size, page_stride);
   else
     return ZA_ERR_UNSUPPORTED;
@@ -118,7 +121,8 @@ template <typename T>
 __global__ void __launch_bounds__(256)
 rotate_part_kernel(const T* __restrict__ src, int src_ld, int src_col, T* __restrict__ dst,
                    int dst_ld, int dst_col, int H, int Dr, const int* __restrict__ positions,
-                   const float* __restrict__ inv_freq, int rot_dims, int adjacent, size_t total) {
+                   const float* __restrict__ inv_freq, int rot_dims, int adjacent, float magnitude,
+                   size_t total) {
   const size_t idx = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   if (idx >= total) return;
   const int per = Dr - rot_dims / 2;         // pairs, then the elements that pass unchanged
@@ -131,6 +135,8 @@ rotate_part_kernel(const T* __restrict__ src, int src_ld, int src_col, T* __rest
     const int a = adjacent ? 2 * i : i, b = adjacent ? 2 * i + 1 : i + half;
     float sn, cs;
     sincosf((float)positions[th / H] * inv_freq[i], &sn, &cs);
+    sn *= magnitude;
+    cs *= magnitude;
     const float u = to_f32<T>(s[a]), v = to_f32<T>(s[b]);
     d[a] = from_f32<T>(u * cs - v * sn);
     d[b] = from_f32<T>(v * cs + u * sn);
@@ -143,7 +149,7 @@ rotate_part_kernel(const T* __restrict__ src, int src_ld, int src_col, T* __rest
 extern "C" int za_rotate_part(const void* src, int dtype, int src_ld, int src_col, void* dst,
                               int dst_ld, int dst_col, int n_tokens, int heads, int rot_dim,
                               const int* positions, const float* inv_freq, int rot_dims,
-                              int adjacent, hipStream_t stream) {
+                              int adjacent, float magnitude, hipStream_t stream) {
   if (n_tokens == 0 || rot_dim == 0) return 0;
   if (n_tokens < 0 || heads <= 0 || rot_dim < 0 || rot_dims < 0 || rot_dims > rot_dim ||
       rot_dims % 2 != 0 || !src || !dst || src_col < 0 || dst_col < 0 ||
@@ -155,11 +161,11 @@ extern "C" int za_rotate_part(const void* src, int dtype, int src_ld, int src_co
   if (dtype == 0)
     hipLaunchKernelGGL((rotate_part_kernel<float>), grid, block, 0, stream, (const float*)src,
                        src_ld, src_col, (float*)dst, dst_ld, dst_col, heads, rot_dim, positions,
-                       inv_freq, rot_dims, adjacent, total);
+                       inv_freq, rot_dims, adjacent, magnitude, total);
   else if (dtype == 1)
     hipLaunchKernelGGL((rotate_part_kernel<bf16_t>), grid, block, 0, stream, (const bf16_t*)src,
                        src_ld, src_col, (bf16_t*)dst, dst_ld, dst_col, heads, rot_dim, positions,
-                       inv_freq, rot_dims, adjacent, total);
+                       inv_freq, rot_dims, adjacent, magnitude, total);
   else
     return ZA_ERR_UNSUPPORTED;
   return za_launch_status();

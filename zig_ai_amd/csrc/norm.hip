@@ -7,6 +7,8 @@
 // The residual stream stays in 32-bit; with `write_residual` the sum is stored
 // back so that the next block adds to it.  With `rows` only the listed rows are
 // normalised (the rows whose logits are wanted) and nothing is stored back.
+// Further forms: the embedding with a second table picked by pairs of tokens, a stream that
+// takes its blocks' results with weights, and one that takes them normed.
 // Formula as in /root/reference/src/transformer/norm.zig:6-33 (32-bit sum of
 // squares, weight multiplied after the scale, no bias).
 #include "common.h"
@@ -405,58 +407,176 @@ extern "C" int za_scaled_add_rmsnorm(float* residual, const void* a, float sa, c
 }
 
 // residual += scale * y / sqrt(mean(y^2) + eps) * weight, in 32-bit, in place: something
-// that is normed by itself before it enters the stream.  A row of up to 256 * NA_VPT
-// elements stays in registers between the sum of squares and the addition.
-#define NA_VPT 16
-template <typename TD>
+// that is normed by itself before it enters the stream.  `y` may be a stack of partial sums
+// (see delta_at).  With `copy` the sum is also stored there, rounded to the type that the
+// next part reads.
+template <typename TD, typename TC>
 __global__ void __launch_bounds__(256)
-normed_add_kernel(float* __restrict__ residual, const TD* __restrict__ y,
-                  const float* __restrict__ weight, int width, float eps, float scale) {
+normed_add_kernel(float* __restrict__ residual, const TD* __restrict__ y, int n_partials,
+                  size_t partial_stride, const float* __restrict__ weight, TC* __restrict__ copy,
+                  int width, float eps, float scale) {
   __shared__ float scratch[16];
   const size_t r = blockIdx.x;
   float* x = residual + r * width;
   const TD* yr = y + r * width;
+  TC* c = copy ? copy + r * width : nullptr;
   const int bd = blockDim.x;
   float ss = 0.f;
-  if (width <= bd * NA_VPT) {
-    float v[NA_VPT];
-#pragma unroll
-    for (int k = 0; k < NA_VPT; ++k) {
-      const int i = threadIdx.x + k * bd;
-      v[k] = i < width ? to_f32<TD>(yr[i]) : 0.f;
-      ss += v[k] * v[k];
-    }
-    ss = block_sum(ss, scratch);
-    const float f = scale / sqrtf(ss / (float)width + eps);
-#pragma unroll
-    for (int k = 0; k < NA_VPT; ++k) {
-      const int i = threadIdx.x + k * bd;
-      if (i < width) x[i] = fmaf(v[k] * f, weight[i], x[i]);
-    }
-    return;
-  }
   for (int i = threadIdx.x; i < width; i += bd) {
-    const float v = to_f32<TD>(yr[i]);
+    const float v = delta_at<TD>(yr, i, n_partials, partial_stride);
     ss += v * v;
   }
   ss = block_sum(ss, scratch);
   const float f = scale / sqrtf(ss / (float)width + eps);
-  for (int i = threadIdx.x; i < width; i += bd)
-    x[i] = fmaf(to_f32<TD>(yr[i]) * f, weight[i], x[i]);
+  for (int i = threadIdx.x; i < width; i += bd) {
+    const float h = fmaf(delta_at<TD>(yr, i, n_partials, partial_stride) * f, weight[i], x[i]);
+    x[i] = h;
+    if (c) c[i] = from_f32<TC>(h);
+  }
 }
 
-extern "C" int za_normed_add(float* residual, const void* y, int y_dtype, const float* weight,
-                             int n_rows, int width, float eps, float scale, hipStream_t stream) {
+// The same for rows of at most 256 * 4 * VPT elements with width % 4 == 0: four elements
+// at a time, everything requested at once, one pass over memory.
+template <typename TD, typename TC, int VPT>
+__global__ void __launch_bounds__(256)
+normed_add_regs_kernel(float* __restrict__ residual, const TD* __restrict__ y, int n_partials,
+                       size_t partial_stride, const float* __restrict__ weight,
+                       TC* __restrict__ copy, int width, float eps, float scale) {
+  __shared__ float scratch[16];
+  const size_t r = blockIdx.x;
+  float* x = residual + r * width;
+  const TD* yr = y + r * width;
+  float v[VPT][4], h[VPT][4], w[VPT][4];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < VPT; ++k) {
+    const int i = (threadIdx.x + k * 256) * 4;
+    if (i < width) {
+      load4<float>(x + i, h[k]);
+      load4<float>(weight + i, w[k]);
+      delta4_at<TD>(yr, i, n_partials, partial_stride, v[k]);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss += v[k][e] * v[k][e];
+    }
+  }
+  ss = block_sum(ss, scratch);
+  const float f = scale / sqrtf(ss / (float)width + eps);
+#pragma unroll
+  for (int k = 0; k < VPT; ++k) {
+    const int i = (threadIdx.x + k * 256) * 4;
+    if (i < width) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) h[k][e] = fmaf(v[k][e] * f, w[k][e], h[k][e]);
+      store4<float>(x + i, h[k]);
+      if (copy) store4<TC>(copy + r * width + i, h[k]);
+    }
+  }
+}
+
+// `copy`: null, or [n_rows][width] of `copy_dtype`.
+extern "C" int za_normed_add(float* residual, const void* y, int y_dtype, int n_partials,
+                             long long partial_stride, const float* weight, void* copy,
+                             int copy_dtype, int n_rows, int width, float eps, float scale,
+                             hipStream_t stream) {
   if (n_rows == 0) return 0;
-  if (n_rows < 0 || width <= 0 || !residual || !y || !weight) return ZA_ERR_ARG;
-  dim3 grid(n_rows), block(width <= 256 ? 64 : 256);
-  if (y_dtype == 0)
-    hipLaunchKernelGGL((normed_add_kernel<float>), grid, block, 0, stream, residual,
-                       (const float*)y, weight, width, eps, scale);
-  else if (y_dtype == 1)
-    hipLaunchKernelGGL((normed_add_kernel<bf16_t>), grid, block, 0, stream, residual,
-                       (const bf16_t*)y, weight, width, eps, scale);
-  else
-    return ZA_ERR_UNSUPPORTED;
+  if (n_rows < 0 || width <= 0 || !residual || !y || !weight || n_partials < 1 ||
+      (n_partials > 1 && partial_stride < (long long)n_rows * width))
+    return ZA_ERR_ARG;
+  dim3 grid(n_rows), block(256);
+  const int vpt = width % 4 == 0 ? (width / 4 + 255) / 256 : 0;   // vectors per thread
+#define ZA_NORMED_ADD(KERNEL, TD, TC)                                                          \
+  hipLaunchKernelGGL((KERNEL), grid, block, 0, stream, residual, (const TD*)y, n_partials,     \
+                     (size_t)partial_stride, weight, (TC*)copy, width, eps, scale)
+#define ZA_NORMED_ADD_CASE(DD, TD, CD, TC)                                                     \
+  if (y_dtype == DD && copy_dtype == CD) {                                                     \
+    if (vpt == 1) ZA_NORMED_ADD((normed_add_regs_kernel<TD, TC, 1>), TD, TC);                  \
+    else if (vpt == 2) ZA_NORMED_ADD((normed_add_regs_kernel<TD, TC, 2>), TD, TC);             \
+    else if (vpt >= 3 && vpt <= 4) ZA_NORMED_ADD((normed_add_regs_kernel<TD, TC, 4>), TD, TC); \
+    else ZA_NORMED_ADD((normed_add_kernel<TD, TC>), TD, TC);                                   \
+    return za_launch_status();                                                                 \
+  }
+  ZA_NORMED_ADD_CASE(0, float, 0, float)
+  ZA_NORMED_ADD_CASE(0, float, 1, bf16_t)
+  ZA_NORMED_ADD_CASE(1, bf16_t, 0, float)
+  ZA_NORMED_ADD_CASE(1, bf16_t, 1, bf16_t)
+#undef ZA_NORMED_ADD_CASE
+#undef ZA_NORMED_ADD
+  return ZA_ERR_UNSUPPORTED;
+}
+
+// The rows that open the stream, with what a token and its predecessor pick from a second
+// table added:
+//   out[t] = table[tokens[t]] + pairs[row(t)]
+//   row(t) = (before * mul_prev + tokens[t] * mul_cur) mod buckets,   before: the token ahead
+//            of t in its request; the request's first token (position 0) takes row `buckets`
+// The token ahead of a portion's first comes from the request's state, which afterwards holds
+// the portion's last token.  One workgroup a token; the workgroup of a portion's first token
+// does both, the read before the write, so no other touches the state.  With `copy` the rows are
+// also stored rounded.
+template <typename T, typename TC>
+__global__ void __launch_bounds__(256)
+embed_pairs_kernel(const int* __restrict__ tokens, const T* __restrict__ table,
+                   const T* __restrict__ pairs, const int* __restrict__ positions,
+                   const int* __restrict__ token_seq, const int* __restrict__ seq_start,
+                   const int* __restrict__ slot_id, int* __restrict__ state, long long slot_stride,
+                   long long buckets, long long mul_prev, long long mul_cur,
+                   float* __restrict__ out, TC* __restrict__ copy, int width, int vocab) {
+  __shared__ long long picked;
+  const int t = blockIdx.x;
+  const int tok = tokens[t];
+  if (threadIdx.x == 0) {
+    const int s = token_seq[t], start = seq_start[s];
+    long long before = -1;
+    if (t > start) {
+      before = tokens[t - 1];
+    } else {
+      int* last = state + (size_t)slot_id[s] * slot_stride;
+      if (positions[t] > 0) before = *last;
+      *last = tokens[seq_start[s + 1] - 1];
+    }
+    long long row = -1;
+    if (t == start && positions[t] == 0) row = buckets;
+    else if (before >= 0 && before < vocab && tok >= 0) row = (before * mul_prev + tok * mul_cur) % buckets;
+    picked = row;
+  }
+  __syncthreads();
+  const long long row = picked;
+  float* o = out + (size_t)t * width;
+  TC* c = copy ? copy + (size_t)t * width : nullptr;
+  // (never read outside a table; an id the host failed to reject poisons its row)
+  const bool ok = tok >= 0 && tok < vocab && row >= 0;
+  const T* a = table + (size_t)(ok ? tok : 0) * width;
+  const T* b = pairs + (size_t)(ok ? row : 0) * width;
+  for (int i = threadIdx.x; i < width; i += blockDim.x) {
+    const float h = ok ? to_f32<T>(a[i]) + to_f32<T>(b[i]) : __builtin_nanf("");
+    o[i] = h;
+    if (c) c[i] = from_f32<TC>(h);
+  }
+}
+
+// `table` [vocab][width] and `pairs` [buckets + 1][width] are of one type; `state`: one int a
+// slot, `slot_stride` ints apart.
+extern "C" int za_embed_pairs(const int* tokens, const void* table, const void* pairs,
+                              int table_dtype, const int* positions, const int* token_seq,
+                              const int* seq_start, const int* slot_id, int* state,
+                              long long slot_stride, long long buckets, long long mul_prev,
+                              long long mul_cur, float* out, void* copy, int copy_dtype,
+                              int n_tokens, int width, int vocab, hipStream_t stream) {
+  if (n_tokens == 0) return 0;
+  if (n_tokens < 0 || width <= 0 || vocab <= 0 || buckets <= 0 || mul_prev < 0 || mul_cur < 0 ||
+      mul_prev > 0x7fffffff || mul_cur > 0x7fffffff || slot_stride <= 0 || !tokens || !table ||
+      !pairs || !positions || !token_seq || !seq_start || !slot_id || !state || !out)
+    return ZA_ERR_ARG;
+  dim3 grid(n_tokens), block(256);
+#define ZA_EMBED_PAIRS(T, TC)                                                                  \
+  hipLaunchKernelGGL((embed_pairs_kernel<T, TC>), grid, block, 0, stream, tokens,              \
+                     (const T*)table, (const T*)pairs, positions, token_seq, seq_start, slot_id, \
+                     state, slot_stride, buckets, mul_prev, mul_cur, out, (TC*)copy, width, vocab)
+  if (table_dtype == 0 && copy_dtype == 0) ZA_EMBED_PAIRS(float, float);
+  else if (table_dtype == 0 && copy_dtype == 1) ZA_EMBED_PAIRS(float, bf16_t);
+  else if (table_dtype == 1 && copy_dtype == 0) ZA_EMBED_PAIRS(bf16_t, float);
+  else if (table_dtype == 1 && copy_dtype == 1) ZA_EMBED_PAIRS(bf16_t, bf16_t);
+  else return ZA_ERR_UNSUPPORTED;
+#undef ZA_EMBED_PAIRS
   return za_launch_status();
 }

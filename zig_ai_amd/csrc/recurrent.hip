@@ -9,7 +9,7 @@
 //    afterwards holds the portion's last L - 1 inputs.
 //
 // 2. matrix_recurrence, per (request, head), with a state S of `dk` rows (key
-//    channels) and `dv` columns, in two forms:
+//    channels) and `dv` columns, in these forms:
 //      SSD (state-space duality):   S <- a S + dt * b x^T;          y = S^T c + D x
 //          a = exp(-exp(A_log) * dt), dt = softplus(raw + dt_bias)      (one per head)
 //      gated delta rule:            S <- diag(g) S;  u = beta (v - S^T k);
@@ -20,6 +20,8 @@
 //      fixed decay (retention):      S <- a_h S + k v^T;             o = S^T q
 //          a_h a constant of the head; the SSD walk with dt = 1 and no D, q and k rotated
 //          and k scaled beforehand by retention_prepare
+//      channel decay (gated linear attention):   S <- diag(a) S + k v^T;   o = S^T q
+//          a one number a head and key channel, made from the token by channel_decay_prepare
 //    A column of S never meets another column: P neighbouring lanes that split its rows
 //    keep one column in registers across all tokens of the portion, read it from the
 //    slot at the start and store it at the end.  The slot holds S turned round,
@@ -193,7 +195,14 @@ struct RecurrenceArgs {
                               // raw step sizes (proj, dt_bias, A_log are not read then)
   const int* seq_count;       // [n], or null: the walkers' token counts, where their rows
                               // are given by (start, count) instead of n + 1 starts
+  int decay_col;              // channel decay: the decay of head h and key channel i lies in
+                              // `conv` at decay_col + h*dk + i
 };
+
+// Forms of the walk: SSD and fixed decay, the delta rule, channel decay.
+#define RC_SSD 0
+#define RC_DELTA 1
+#define RC_CHANNEL 2
 
 // Everything of a token that does not depend on the state, for the delta rule: the unit
 // vectors, the decays and the write strengths, once per token instead of once per
@@ -274,15 +283,16 @@ __device__ __forceinline__ float group_sum(float x) {
 // load pattern allows, which leaves LDS for more waves when every portion is a token or two.
 // (LONG == 1: half as long chunks, for steps with more waves than the chip has SIMDs, where
 // LDS decides how many of them run at once)
-template <int P, bool DELTA, int LONG>
+template <int P, int FORM, int LONG>
 __global__ void __launch_bounds__(64, 2)
 matrix_recurrence_kernel(RecurrenceArgs a) {
+  constexpr bool DELTA = FORM == RC_DELTA, CHANNEL = FORM == RC_CHANNEL;
   constexpr int R = RC_ROWS;
   constexpr int DKMAX = R * P;
   constexpr int CH_MIN = 4 * P < 64 ? 64 / (4 * P) : 1;
   constexpr int CH_LONG = (P <= 8 ? 16 : (P == 16 ? 8 : (P == 32 ? 4 : 2))) / (LONG == 1 ? 2 : 1);
   constexpr int CH = LONG ? (CH_LONG < CH_MIN ? CH_MIN : CH_LONG) : (CH_MIN < 2 ? 2 : CH_MIN);
-  constexpr int NV = DELTA ? 3 : 2;                 // vectors of dk floats a token
+  constexpr int NV = DELTA || CHANNEL ? 3 : 2;      // vectors of dk floats a token
   constexpr int KPAD = RC_SHARE * P;
   // a chunk's vectors come four floats a lane and load: LPV lanes cover a vector (or a
   // quarter of a long one), so one load instruction of the wave brings TPL tokens' worth
@@ -313,6 +323,7 @@ matrix_recurrence_kernel(RecurrenceArgs a) {
     stride = a.conv_width;
     base[0] = a.conv + a.k_col + g * dk;
     base[1] = a.conv + a.q_col + g * dk;
+    if (CHANNEL) base[NV - 1] = a.conv + a.decay_col + h * dk;   // decays
   }
   const float* xsrc = a.conv + a.x_col + h * dv + (owner ? col : 0);
 
@@ -336,11 +347,11 @@ matrix_recurrence_kernel(RecurrenceArgs a) {
         if (part * R + r < dk) S[r] = st[r];
     }
   }
-  const bool fixed = !DELTA && a.fixed_decay != nullptr;
+  const bool fixed = FORM == RC_SSD && a.fixed_decay != nullptr;
   const float fixed_a = fixed ? a.fixed_decay[h] : 0.f;
-  const float neg_A = (DELTA || fixed) ? 0.f : -expf(a.A_log[h]);
-  const float Dh = (DELTA || !a.D) ? 0.f : a.D[h];
-  const float dtb = (DELTA || fixed) ? 0.f : a.dt_bias[h];
+  const float neg_A = (FORM != RC_SSD || fixed) ? 0.f : -expf(a.A_log[h]);
+  const float Dh = (FORM != RC_SSD || !a.D) ? 0.f : a.D[h];
+  const float dtb = (FORM != RC_SSD || fixed) ? 0.f : a.dt_bias[h];
 
   // (whole four-float loads need the vectors to start on 16-byte boundaries)
   bool vec_loads = dk % 4 == 0 && stride % 4 == 0;
@@ -358,7 +369,7 @@ matrix_recurrence_kernel(RecurrenceArgs a) {
       const int tt = group * TPL + lane_tt, i = piece * 256 + lane_i;
       // (a chunk's places beyond the portion's end hold tokens that change nothing: no
       // decay, nothing written, nothing read; the walk then needs no conditions)
-      const float idle = (DELTA && v == NV - 1 && c0 + tt >= n) ? 1.f : 0.f;
+      const float idle = (NV == 3 && v == NV - 1 && c0 + tt >= n) ? 1.f : 0.f;
       float4 x = make_float4(idle, idle, idle, idle);
       if (c0 + tt < n && i < dk) {
         const float* src = base[v] + (size_t)(start + c0 + tt) * stride + i;
@@ -382,7 +393,7 @@ matrix_recurrence_kernel(RecurrenceArgs a) {
       const size_t t = start + c0 + lane;
       if (DELTA) {
         snext = a.prep[t * a.prep_width + 2 * a.G * dk + a.H * dk + h];
-      } else if (!fixed) {
+      } else if (FORM == RC_SSD && !fixed) {
         const size_t at = t * a.proj_stride + a.gate_col + h;
         snext = a.proj_bf16 ? (float)((const bf16_t*)a.proj)[at] : ((const float*)a.proj)[at];
       }
@@ -399,7 +410,7 @@ matrix_recurrence_kernel(RecurrenceArgs a) {
     if (lane < CH) {
       if (DELTA) {
         scal[buf][lane][0] = snext;
-      } else {
+      } else if (FORM == RC_SSD) {
         const float dt = fixed ? 1.f : softplus_f(snext + dtb);
         scal[buf][lane][0] = lane < chunk_left ? (fixed ? fixed_a : expf(neg_A * dt)) : 1.f;
         scal[buf][lane][1] = lane < chunk_left ? dt : 0.f;
@@ -464,6 +475,22 @@ matrix_recurrence_kernel(RecurrenceArgs a) {
             a3 = fmaf(S[r + 3], qq[r + 3], a3);
           }
           o = group_sum<P>((a0 + a1) + (a2 + a3));
+        } else if (CHANNEL) {
+          float a0 = 0.f, a1 = 0.f, a2 = 0.f, a3 = 0.f;
+#pragma unroll
+          for (int r = 0; r < R; r += 4) {
+            const float4 g4 =
+                *reinterpret_cast<const float4*>(&vecs[buf][tt][NV - 1][part * RC_SHARE + r]);
+            S[r] = fmaf(g4.x, S[r], xv * kk[r]);
+            S[r + 1] = fmaf(g4.y, S[r + 1], xv * kk[r + 1]);
+            S[r + 2] = fmaf(g4.z, S[r + 2], xv * kk[r + 2]);
+            S[r + 3] = fmaf(g4.w, S[r + 3], xv * kk[r + 3]);
+            a0 = fmaf(S[r], qq[r], a0);
+            a1 = fmaf(S[r + 1], qq[r + 1], a1);
+            a2 = fmaf(S[r + 2], qq[r + 2], a2);
+            a3 = fmaf(S[r + 3], qq[r + 3], a3);
+          }
+          o = group_sum<P>((a0 + a1) + (a2 + a3));
         } else {
           const float decay_t = scal[buf][tt][0], dtx = scal[buf][tt][1] * xv;
           float a0 = 0.f, a1 = 0.f, a2 = 0.f, a3 = 0.f;
@@ -509,7 +536,7 @@ matrix_recurrence_kernel(RecurrenceArgs a) {
   }
 }
 
-template <bool DELTA>
+template <int FORM>
 static int launch_recurrence(const RecurrenceArgs& a, int n_seqs, int P, bool long_portions,
                              hipStream_t stream) {
   dim3 grid(n_seqs, a.H, (a.dv * P + 63) / 64), block(64);
@@ -518,11 +545,11 @@ static int launch_recurrence(const RecurrenceArgs& a, int n_seqs, int P, bool lo
 #define ZA_RECURRENCE(PP)                                                                      \
   case PP:                                                                                     \
     if (long_portions && crowded)                                                              \
-      hipLaunchKernelGGL((matrix_recurrence_kernel<PP, DELTA, 1>), grid, block, 0, stream, a); \
+      hipLaunchKernelGGL((matrix_recurrence_kernel<PP, FORM, 1>), grid, block, 0, stream, a); \
     else if (long_portions)                                                                    \
-      hipLaunchKernelGGL((matrix_recurrence_kernel<PP, DELTA, 2>), grid, block, 0, stream, a); \
+      hipLaunchKernelGGL((matrix_recurrence_kernel<PP, FORM, 2>), grid, block, 0, stream, a); \
     else                                                                                       \
-      hipLaunchKernelGGL((matrix_recurrence_kernel<PP, DELTA, 0>), grid, block, 0, stream, a); \
+      hipLaunchKernelGGL((matrix_recurrence_kernel<PP, FORM, 0>), grid, block, 0, stream, a); \
     break
   switch (P) {
     ZA_RECURRENCE(1);
@@ -569,10 +596,10 @@ extern "C" int za_matrix_recurrence(int form, int dtype, const float* conv, int 
   RecurrenceArgs a{conv, conv_width, q_col, k_col, x_col, proj, proj_stride, gate_col, dtype,
                    prep, prep_width, dt_bias, A_log, form == 2 ? nullptr : D, state, slot_stride,
                    seq_start, slot_id, out, H, G, dk, dv,
-                   form == 2 ? (const float*)decay : nullptr, nullptr};
+                   form == 2 ? (const float*)decay : nullptr, nullptr, 0};
   // (a function of the step's shape alone, as a recorded step needs it)
   const bool long_portions = n_tokens > 4 * n_seqs;
-  if (form != 1) return launch_recurrence<false>(a, n_seqs, lanes, long_portions, stream);
+  if (form != 1) return launch_recurrence<RC_SSD>(a, n_seqs, lanes, long_portions, stream);
   const dim3 prep_grid(n_tokens, 2 * G + (H * dk + 255) / 256);
   if (dtype == 0)
     hipLaunchKernelGGL((delta_prepare_kernel<float>), prep_grid, dim3(64), 0, stream, conv,
@@ -586,7 +613,7 @@ extern "C" int za_matrix_recurrence(int form, int dtype, const float* conv, int 
                        dk);
   const int rc = za_launch_status();
   if (rc != 0) return rc;
-  return launch_recurrence<true>(a, n_seqs, lanes, long_portions, stream);
+  return launch_recurrence<RC_DELTA>(a, n_seqs, lanes, long_portions, stream);
 }
 
 // ------------------------------------------------- fixed decay, long portions in chunks
@@ -710,8 +737,8 @@ extern "C" int za_retention_chunked(const float* vectors, int width, int q_col, 
   const long long elems = (long long)H * dk * dv;
   RecurrenceArgs a{vectors, width, q_col, k_col, x_col, nullptr, 0, 0, 0, nullptr, 0, nullptr,
                    nullptr, nullptr, chunk_state, elems, item_row0, iota, out, H, H, dk, dv,
-                   decay, item_count};
-  int rc = launch_recurrence<false>(a, n_items, lanes, n_tokens > 4 * n_items, stream);
+                   decay, item_count, 0};
+  int rc = launch_recurrence<RC_SSD>(a, n_items, lanes, n_tokens > 4 * n_items, stream);
   if (rc != 0) return rc;
   hipLaunchKernelGGL(chunk_state_prefix_kernel, dim3(n_seqs, (unsigned)((elems + 255) / 256)),
                      dim3(256), 0, stream, chunk_state, state, slot_stride, slot_id, item_seq,
@@ -728,6 +755,298 @@ extern "C" int za_retention_chunked(const float* vectors, int width, int q_col, 
     hipLaunchKernelGGL((chunk_correct_kernel<128>), grid, dim3(128), 0, stream, vectors, width,
                        q_col, chunk_state, item_row0, item_count, decay, out, H, dk, dv,
                        tokens_per_block);
+  return za_launch_status();
+}
+
+// ------------------------------------------------------ a decay a head and key channel
+// What the channel-decay walk reads, from the opening projection's rows, per token as 32-bit
+// floats
+//   out[t] = [q * q_scale: H*dk | k: H*dk | a: H*dk | v: H*dv]  (padded to `out_width`)
+// with the decays a = sigmoid(z)^(1/root), z = up low[t] + bias: `low` the token's `rank` columns
+// of the projection, `up` [H*dk][rank] a second, small product taken here in 32-bit.  The power
+// is taken through the logarithm, log sigmoid(z) = -softplus(-z).
+// grid (tokens / GP_TOKENS, 256 channels).
+#define GP_TOKENS 8
+#define GP_RANK 256     // columns of `low` staged at a time
+template <typename T, typename TW>
+__global__ void __launch_bounds__(256)
+channel_decay_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_col, int k_col,
+                             int v_col, int low_col, int rank, const TW* __restrict__ up,
+                             const float* __restrict__ bias, float inv_root, float q_scale,
+                             float* __restrict__ out, int out_width, int n_tokens, int hk, int hv) {
+  __shared__ float low[GP_TOKENS][GP_RANK];
+  const int t0 = blockIdx.x * GP_TOKENS, c = blockIdx.y * 256 + threadIdx.x;
+  const int nt = n_tokens - t0 < GP_TOKENS ? n_tokens - t0 : GP_TOKENS;
+  float z[GP_TOKENS];
+#pragma unroll
+  for (int i = 0; i < GP_TOKENS; ++i) z[i] = 0.f;
+  for (int r0 = 0; r0 < rank; r0 += GP_RANK) {
+    const int rn = rank - r0 < GP_RANK ? rank - r0 : GP_RANK;
+    __syncthreads();
+    for (int idx = threadIdx.x; idx < GP_TOKENS * rn; idx += 256) {
+      const int i = idx / rn, r = idx % rn;
+      low[i][r] = i < nt ? to_f32<T>(proj[(size_t)(t0 + i) * proj_stride + low_col + r0 + r]) : 0.f;
+    }
+    __syncthreads();
+    if (c < hk) {
+      const TW* w = up + (size_t)c * rank + r0;
+      for (int r = 0; r < rn; ++r) {
+        const float wv = to_f32<TW>(w[r]);
+#pragma unroll
+        for (int i = 0; i < GP_TOKENS; ++i) z[i] = fmaf(wv, low[i][r], z[i]);
+      }
+    }
+  }
+  const float b = c < hk ? bias[c] : 0.f;
+#pragma unroll
+  for (int i = 0; i < GP_TOKENS; ++i) {
+    if (i >= nt) continue;
+    const T* row = proj + (size_t)(t0 + i) * proj_stride;
+    float* dst = out + (size_t)(t0 + i) * out_width;
+    if (c < hk) {
+      dst[c] = to_f32<T>(row[q_col + c]) * q_scale;
+      dst[hk + c] = to_f32<T>(row[k_col + c]);
+      dst[2 * hk + c] = expf(-softplus_f(-(z[i] + b)) * inv_root);
+    }
+    if (c < hv) dst[3 * hk + c] = to_f32<T>(row[v_col + c]);
+  }
+}
+
+extern "C" int za_channel_decay_prepare(const void* proj, int dtype, int proj_stride, int q_col,
+                                        int k_col, int v_col, int low_col, int rank,
+                                        const void* up, int up_dtype, const float* bias, float root,
+                                        float q_scale, float* out, int out_width, int n_tokens,
+                                        int H, int dk, int dv, hipStream_t stream) {
+  if (n_tokens == 0) return 0;
+  if (n_tokens < 0 || H <= 0 || dk <= 0 || dv <= 0 || rank <= 0 || !(root > 0.f) || !proj || !up ||
+      !bias || !out || q_col < 0 || k_col < 0 || v_col < 0 || low_col < 0 ||
+      q_col + H * dk > proj_stride || k_col + H * dk > proj_stride ||
+      v_col + H * dv > proj_stride || low_col + rank > proj_stride ||
+      out_width < 3 * H * dk + H * dv)
+    return ZA_ERR_ARG;
+  const int hk = H * dk, hv = H * dv, most = hk > hv ? hk : hv;
+  dim3 grid((n_tokens + GP_TOKENS - 1) / GP_TOKENS, (most + 255) / 256), block(256);
+#define ZA_CDP(T, TW)                                                                          \
+  hipLaunchKernelGGL((channel_decay_prepare_kernel<T, TW>), grid, block, 0, stream,            \
+                     (const T*)proj, proj_stride, q_col, k_col, v_col, low_col, rank,          \
+                     (const TW*)up, bias, 1.0f / root, q_scale, out, out_width, n_tokens, hk, hv)
+  if (dtype == 0 && up_dtype == 0) ZA_CDP(float, float);
+  else if (dtype == 1 && up_dtype == 1) ZA_CDP(bf16_t, bf16_t);
+  else if (dtype == 1 && up_dtype == 0) ZA_CDP(bf16_t, float);
+  else return ZA_ERR_UNSUPPORTED;
+#undef ZA_CDP
+  return za_launch_status();
+}
+
+// The plain walk with these vectors (`vectors` as channel_decay_prepare leaves them).
+extern "C" int za_channel_recurrence(const float* vectors, int width, float* state,
+                                     long long slot_stride, const int* seq_start,
+                                     const int* slot_id, float* out, int n_tokens, int n_seqs, int H,
+                                     int dk, int dv, int lanes, hipStream_t stream) {
+  if (n_tokens == 0 || n_seqs == 0) return 0;
+  if (n_tokens < 0 || n_seqs < 0 || H <= 0 || dk <= 0 || dv <= 0 || !vectors || !state ||
+      !seq_start || !slot_id || !out || width < 3 * H * dk + H * dv || lanes < 1 || lanes > 64 ||
+      (lanes & (lanes - 1)) || lanes * RC_ROWS < dk || slot_stride < (long long)H * dk * dv)
+    return ZA_ERR_ARG;
+  const int hk = H * dk;
+  RecurrenceArgs a{vectors, width, 0, hk, 3 * hk, nullptr, 0, 0, 0, nullptr, 0, nullptr, nullptr,
+                   nullptr, state, slot_stride, seq_start, slot_id, out, H, H, dk, dv, nullptr,
+                   nullptr, 2 * hk};
+  return launch_recurrence<RC_CHANNEL>(a, n_seqs, lanes, n_tokens > 4 * n_seqs, stream);
+}
+
+// Long portions in chunks, as for the fixed decay: every chunk is walked by itself from an
+// empty state, and what the state before it adds to its read-outs is linear in that state:
+//   1. the walk, one walker a chunk:              o_local[t], the chunk's own final state L_c
+//   2. channel_scan: with A_t the product of the chunk's decays up to and including token t
+//      (at most one, so nothing overflows),       q_t <- q_t * A_t in place;  A_c = A at its end
+//   3. channel_prefix: the state before chunk c,  B_c = diag(A_(c-1)) B_(c-1) + L_(c-1)
+//   4. channel_readout:                           o[t] = o_local[t] + B_c^T (q_t * A_t)
+// 4 is a matrix product and runs on the matrix cores in their 32-bit form
+// (v_mfma_f32_16x16x4_f32: products and sums in full 32-bit).
+
+// A workgroup serves 64 channels of one chunk: 8 waves take an eighth of its tokens each
+// (at most CS_PART), their decays kept in registers between the product and the scaling.
+#define CS_PART 32
+__global__ void __launch_bounds__(512)
+channel_scan_kernel(float* __restrict__ vectors, int width, const int* __restrict__ item_row0,
+                    const int* __restrict__ item_count, float* __restrict__ total, int hk) {
+  __shared__ float part_total[8][64];
+  const int item = blockIdx.x, lane = threadIdx.x & 63, part = threadIdx.x >> 6;
+  const int c = blockIdx.y * 64 + lane;
+  const int row0 = item_row0[item], cnt = item_count[item];
+  const int per = (cnt + 7) / 8, begin = part * per;
+  const int n = cnt - begin < per ? cnt - begin : per;      // (may be negative: no tokens)
+  float* base = vectors + (size_t)(row0 + begin) * width + c;
+  float a[CS_PART];
+  float prod = 1.f;
+#pragma unroll
+  for (int j = 0; j < CS_PART; ++j) a[j] = (c < hk && j < n) ? base[(size_t)j * width + 2 * hk] : 1.f;
+#pragma unroll
+  for (int j = 0; j < CS_PART; ++j) prod *= a[j];
+  part_total[part][lane] = prod;
+  __syncthreads();
+  float before = 1.f, all = 1.f;
+#pragma unroll
+  for (int p = 0; p < 8; ++p) {
+    if (p < part) before *= part_total[p][lane];
+    all *= part_total[p][lane];
+  }
+  if (c >= hk) return;
+  if (part == 0) total[(size_t)item * hk + c] = all;
+#pragma unroll
+  for (int j0 = 0; j0 < CS_PART; j0 += 8) {
+    float q[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) q[j] = j0 + j < n ? base[(size_t)(j0 + j) * width] : 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      before *= a[j0 + j];
+      if (j0 + j < n) base[(size_t)(j0 + j) * width] = q[j] * before;
+    }
+  }
+}
+
+// One thread a state element; the chunks of a request are neighbours in the list.
+__global__ void __launch_bounds__(256)
+channel_prefix_kernel(float* __restrict__ chunk_state, float* __restrict__ state,
+                      long long slot_stride, const int* __restrict__ slot_id,
+                      const int* __restrict__ item_seq, int n_items,
+                      const float* __restrict__ total, int elems, int hk, int dk, int dv) {
+  __shared__ int bounds[2];
+  const int s = blockIdx.x, e = blockIdx.y * 256 + threadIdx.x;
+  if (threadIdx.x == 0) { bounds[0] = n_items; bounds[1] = 0; }
+  __syncthreads();
+  for (int i = threadIdx.x; i < n_items; i += 256)
+    if (item_seq[i] == s) {
+      atomicMin(&bounds[0], i);
+      atomicMax(&bounds[1], i + 1);
+    }
+  __syncthreads();
+  if (e >= elems) return;
+  const int first = bounds[0], last = bounds[1];
+  const int channel = e / (dk * dv) * dk + e % dk;
+  float* slot = state + (size_t)slot_id[s] * slot_stride + e;
+  float S = *slot;
+  for (int i0 = first; i0 < last; i0 += 8) {
+    float local[8], a[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const bool in = i0 + j < last;
+      local[j] = in ? chunk_state[(size_t)(i0 + j) * elems + e] : 0.f;
+      a[j] = in ? total[(size_t)(i0 + j) * hk + channel] : 1.f;
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      if (i0 + j < last) chunk_state[(size_t)(i0 + j) * elems + e] = S;
+      S = fmaf(a[j], S, local[j]);
+    }
+  }
+  *slot = S;
+}
+
+// Four consecutive floats, those at and beyond `n` as zeros.
+__device__ __forceinline__ f32x4_t four_or_fewer(const float* p, int n, bool aligned) {
+  f32x4_t v = {0.f, 0.f, 0.f, 0.f};
+  if (aligned && n >= 4) return *reinterpret_cast<const f32x4_t*>(p);
+#pragma unroll
+  for (int j = 0; j < 4; ++j)
+    if (j < n) v[j] = p[j];
+  return v;
+}
+
+// grid (items, heads, tokens / 64 * columns / 64); four waves of 16 tokens x 64 columns.
+// Operand layout of v_mfma_f32_16x16x4_f32: lane l supplies row (l % 16), k-slot (l / 16) of
+// either operand and receives rows (l / 16) * 4 .. + 3, column (l % 16).  The order in which k
+// runs is free as long as both operands agree: slot g of step j is channel 4 g + j of a
+// block of 16, so that a lane's four steps are four neighbouring floats.
+__global__ void __launch_bounds__(256)
+channel_readout_kernel(const float* __restrict__ vectors, int width,
+                       const float* __restrict__ chunk_state, const int* __restrict__ item_row0,
+                       const int* __restrict__ item_count, float* __restrict__ out, int H, int dk,
+                       int dv, int column_blocks) {
+  const int item = blockIdx.x, h = blockIdx.y;
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  const int r16 = lane & 15, g = lane >> 4;
+  const int row0 = item_row0[item], cnt = item_count[item];
+  const int t0 = (blockIdx.z / column_blocks) * 64 + wave * 16;
+  const int n0 = (blockIdx.z % column_blocks) * 64;
+  if (t0 >= cnt) return;
+  const bool row_ok = t0 + r16 < cnt;
+  const float* q = vectors + (size_t)(row0 + (row_ok ? t0 + r16 : 0)) * width + h * dk;
+  const float* B = chunk_state + ((size_t)item * H + h) * dv * dk;
+  const bool aligned = dk % 4 == 0 && width % 4 == 0;
+  f32x4_t acc[4];
+#pragma unroll
+  for (int j = 0; j < 4; ++j) acc[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 0; k0 < dk; k0 += 16) {
+    const int k = k0 + 4 * g, left = dk - k;
+    const f32x4_t fq = row_ok ? four_or_fewer(q + k, left, aligned) : f32x4_t{0.f, 0.f, 0.f, 0.f};
+    f32x4_t fb[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int n = n0 + j * 16 + r16;
+      fb[j] = n < dv ? four_or_fewer(B + (size_t)n * dk + k, left, aligned)
+                     : f32x4_t{0.f, 0.f, 0.f, 0.f};
+    }
+#pragma unroll
+    for (int step = 0; step < 4; ++step)
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        acc[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(fq[step], fb[j][step], acc[j], 0, 0, 0);
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int t = t0 + g * 4 + i;
+    if (t >= cnt) continue;
+    float* o = out + (size_t)(row0 + t) * H * dv + h * dv;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const int n = n0 + j * 16 + r16;
+      if (n < dv) o[n] += acc[j][i];
+    }
+  }
+}
+
+// `item_*`: the step's work items of at most `chunk` (<= 8 * CS_PART) rows; `iota`: 0 .. n_items
+// - 1; `chunk_state`: n_items * H*dv*dk floats, zero on entry; `total`: n_items * H*dk floats.
+// `vectors`' queries are overwritten.
+extern "C" int za_channel_recurrence_chunked(float* vectors, int width, float* state,
+                                             long long slot_stride, const int* slot_id,
+                                             const int* item_seq, const int* item_row0,
+                                             const int* item_count, const int* iota, int n_items,
+                                             int n_seqs, int chunk, float* chunk_state,
+                                             float* total, float* out, int n_tokens, int H, int dk,
+                                             int dv, int lanes, hipStream_t stream) {
+  if (n_tokens == 0 || n_items == 0) return 0;
+  if (n_tokens < 0 || n_seqs <= 0 || n_items < n_seqs || chunk <= 0 || H <= 0 || dk <= 0 ||
+      dv <= 0 || !vectors || !state || !slot_id || !item_seq || !item_row0 || !item_count ||
+      !iota || !chunk_state || !total || !out || width < 3 * H * dk + H * dv || lanes < 1 ||
+      lanes > 64 || (lanes & (lanes - 1)) || lanes * RC_ROWS < dk ||
+      slot_stride < (long long)H * dk * dv)
+    return ZA_ERR_ARG;
+  if (chunk > 8 * CS_PART || (long long)H * dk * dv > 0x7fffffffLL) return ZA_ERR_UNSUPPORTED;
+  const int hk = H * dk;
+  const long long elems = (long long)hk * dv;
+  RecurrenceArgs a{vectors, width, 0, hk, 3 * hk, nullptr, 0, 0, 0, nullptr, 0, nullptr, nullptr,
+                   nullptr, chunk_state, elems, item_row0, iota, out, H, H, dk, dv, nullptr,
+                   item_count, 2 * hk};
+  int rc = launch_recurrence<RC_CHANNEL>(a, n_items, lanes, n_tokens > 4 * n_items, stream);
+  if (rc != 0) return rc;
+  hipLaunchKernelGGL(channel_scan_kernel, dim3(n_items, (hk + 63) / 64), dim3(512), 0, stream,
+                     vectors, width, item_row0, item_count, total, hk);
+  rc = za_launch_status();
+  if (rc != 0) return rc;
+  hipLaunchKernelGGL(channel_prefix_kernel, dim3(n_seqs, (unsigned)((elems + 255) / 256)),
+                     dim3(256), 0, stream, chunk_state, state, slot_stride, slot_id, item_seq,
+                     n_items, total, (int)elems, hk, dk, dv);
+  rc = za_launch_status();
+  if (rc != 0) return rc;
+  const int column_blocks = (dv + 63) / 64;
+  hipLaunchKernelGGL(channel_readout_kernel,
+                     dim3(n_items, H, (unsigned)((chunk + 63) / 64 * column_blocks)), dim3(256), 0,
+                     stream, vectors, width, chunk_state, item_row0, item_count, out, H, dk, dv,
+                     column_blocks);
   return za_launch_status();
 }
 

@@ -60,6 +60,9 @@ class StepContext:
     # diagnostics: when a dict, the part that is running may leave copies of its
     # intermediate tensors in it by name (token rows first); see DecoderModel.forward
     taps: Optional[Dict[str, torch.Tensor]] = None
+    # the residual stream rounded to the run's type, when the kernel that wrote the stream last
+    # left such a copy; the model drops it as soon as anything else touches the stream
+    rounded: Optional[torch.Tensor] = None
 
     def attention_items(self, rows_per_item: int):
         """Work items of at most ``rows_per_item`` consecutive query rows of one

@@ -18,6 +18,8 @@ from ..parts import base as parts
 from ..weights.loader import load_tensors
 from .batch import StepContext
 
+EMBEDDING_CACHE = "embedding"      # the embedding's entry among the cache needs
+
 _RUN_DTYPES = {"bfloat16": torch.bfloat16, "bf16": torch.bfloat16,
                "float32": torch.float32, "fp32": torch.float32, "f32": torch.float32}
 
@@ -128,6 +130,12 @@ class DecoderModel:
                         f"run-order entries sharing cache {key} need different caches: "
                         f"{self.cache_needs[key]} and {need}")
                 self.cache_needs[key] = need
+        # an embedding that keeps something a request (its last token, say)
+        need = getattr(parts.lookup("embedding", spec.embedding.kind), "cache_need", None)
+        need = need(spec.embedding.params) if need is not None else None
+        self.embedding_keeps = need is not None
+        if self.embedding_keeps:
+            self.cache_needs[EMBEDDING_CACHE] = need
         writers = {key for c in self.schedule if c.writes_cache for key, _ in self.cache_keys(c)}
         for call in self.schedule:
             for key, _ in self.cache_keys(call):
@@ -223,7 +231,8 @@ class DecoderModel:
     def cache_views(self, cache: CacheManager) -> List[Any]:
         """Per run-order entry what its block's ``forward`` receives as ``cache``: the
         mixer's view, or for a block with several mixers (or none) a dictionary from
-        the mixers' names to their views."""
+        the mixers' names to their views.  Behind them, for an embedding that keeps
+        something a request, the embedding's view."""
         out = []
         for call in self.schedule:
             keys = self.cache_keys(call)
@@ -231,6 +240,8 @@ class DecoderModel:
                 out.append(cache.view(call.cache, call.writes_cache))
             else:
                 out.append({name: cache.view(key, call.writes_cache) for key, name in keys})
+        if self.embedding_keeps:
+            out.append(cache.view(EMBEDDING_CACHE))
         return out
 
     # ------------------------------------------------------------------ forward
@@ -248,7 +259,9 @@ class DecoderModel:
 
     def _forward(self, step: StepContext, views: Sequence[CacheView],
                  taps: Optional[List[Dict[str, torch.Tensor]]]) -> torch.Tensor:
-        residual = self.embedding.forward(step.token_ids)
+        step.rounded = None
+        residual = self.embedding.forward(step.token_ids, step, views[len(self.schedule)]) \
+            if self.embedding_keeps else self.embedding.forward(step.token_ids)
         pending = None
         if taps is not None:
             taps.append({"stream": residual.clone()})
@@ -260,9 +273,13 @@ class DecoderModel:
         for call, view in zip(self.schedule, views):
             step.taps = {} if taps is not None else None
             if call.before is not None:
+                step.rounded = None
                 residual, pending = self.stream_parts[call.before.part].forward(
                     residual, pending, origin, step, **dict(call.before.args))
-            residual, pending = self.blocks[call.layer].forward(residual, pending, step, view)
+            block = self.blocks[call.layer]
+            residual, pending = block.forward(residual, pending, step, view)
+            if call.after is not None or not getattr(block, "leaves_rounded", False):
+                step.rounded = None
             if call.after is not None:
                 residual, pending = self.stream_parts[call.after.part].forward(
                     residual, pending, origin, step, **dict(call.after.args))
@@ -272,7 +289,7 @@ class DecoderModel:
                     now += (pending.sum(dim=0) if pending.dim() == 3 else pending).float()
                 step.taps["stream"] = now
                 taps.append(step.taps)
-        step.taps = None
+        step.taps = step.rounded = None
         if step.n_logit_rows == 0:
             return torch.empty((0, self.spec.vocab_size), dtype=torch.float32,
                                device=self.runtime.device)

@@ -100,8 +100,8 @@ _SIGNATURES = {
                                                 c_void_p, c_int, c_int, c_float, c_void_p],
     ("attention", "za_head_gate"): [c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
                                     c_float, c_void_p],
-    ("activation", "za_clamped_glu"): [c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_float,
-                                       c_float, c_void_p],
+    ("activation", "za_clamped_glu"): [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_float,
+                                       c_float, c_float, c_void_p],
     ("norm", "za_scaled_add_rmsnorm"): [c_void_p, c_void_p, c_float, c_void_p, c_float, c_int,
                                         c_void_p, c_void_p, c_int, c_int, c_int, c_float, c_void_p],
     ("recurrent", "za_causal_conv_silu"): [c_void_p, c_int, c_int, c_int, c_void_p, c_void_p,
@@ -165,19 +165,33 @@ _SIGNATURES = {
     ("activation", "za_softcap"): [c_void_p, c_float, c_longlong, c_void_p],
     ("activation", "za_table_gate"): [c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int,
                                       c_int, c_void_p, c_int, c_int, c_int, c_void_p],
-    ("norm", "za_normed_add"): [c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_float,
-                                c_float, c_void_p],
+    ("norm", "za_normed_add"): [c_void_p, c_void_p, c_int, c_int, c_longlong, c_void_p, c_void_p,
+                                c_int, c_int, c_int, c_float, c_float, c_void_p],
+    ("norm", "za_embed_pairs"): [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
+                                 c_void_p, c_void_p, c_longlong, c_longlong, c_longlong, c_longlong,
+                                 c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
+    ("recurrent", "za_channel_decay_prepare"): [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
+                                                c_int, c_void_p, c_int, c_void_p, c_float, c_float,
+                                                c_void_p, c_int, c_int, c_int, c_int, c_int,
+                                                c_void_p],
+    ("recurrent", "za_channel_recurrence"): [c_void_p, c_int, c_void_p, c_longlong, c_void_p,
+                                             c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
+                                             c_int, c_void_p],
+    ("recurrent", "za_channel_recurrence_chunked"): [c_void_p, c_int, c_void_p, c_longlong, c_void_p,
+                                                     c_void_p, c_void_p, c_void_p, c_void_p, c_int,
+                                                     c_int, c_int, c_void_p, c_void_p, c_void_p,
+                                                     c_int, c_int, c_int, c_int, c_int, c_void_p],
     ("experts", "za_route_topk"): [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int,
                                    c_float, c_int, c_int, c_void_p, c_void_p, c_void_p],
     ("experts", "za_experts_combine"): [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
                                         c_void_p, c_void_p, c_int, c_void_p, c_int, c_int, c_int,
-                                        c_int, c_void_p],
+                                        c_int, c_int, c_void_p],
     ("latent", "za_latent_prepare"): [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int,
                                       c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_void_p,
-                                      c_int, c_int, c_void_p, c_void_p, c_int, c_longlong, c_int,
-                                      c_void_p],
+                                      c_int, c_int, c_float, c_void_p, c_void_p, c_int, c_longlong,
+                                      c_int, c_void_p],
     ("latent", "za_rotate_part"): [c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_int, c_int,
-                                   c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p],
+                                   c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_float, c_void_p],
     ("latent", "za_head_linear"): [c_void_p, c_int, c_int, c_int, c_void_p, c_int, c_void_p, c_int,
                                    c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int, c_int,
                                    c_int, c_void_p],
@@ -322,6 +336,45 @@ def embed_gather(tokens: torch.Tensor, table: torch.Tensor) -> torch.Tensor:
                                         tokens.numel(), width, vocab, _stream())
     _check(rc, "embed_gather")
     return out
+
+
+def embed_pairs(tokens: torch.Tensor, table: torch.Tensor, pairs: torch.Tensor,
+                positions: torch.Tensor, token_seq: torch.Tensor, seq_start: torch.Tensor,
+                slot_id: torch.Tensor, state: torch.Tensor, mul_prev: int, mul_cur: int,
+                copy_dtype: Optional[torch.dtype] = None):
+    """``table[tokens[t]] + pairs[row(t)]`` as 32-bit rows, ``row(t) = (before * mul_prev +
+    tokens[t] * mul_cur) mod buckets`` with ``before`` the token ahead of ``t`` in its request
+    (``pairs`` has ``buckets + 1`` rows; a request's first token takes the last).  ``state``
+    (int32 ``[slots, 1]``, slots any distance apart) holds every request's last token and is brought up
+    to date.  Returns ``(rows, copy)``: ``copy`` the rows rounded to ``copy_dtype``, or None."""
+    _need(tokens, "tokens", torch.int32)
+    _need(table, "table", (torch.float32, torch.bfloat16))
+    if tokens.dim() != 1 or table.dim() != 2:
+        raise KernelError("embed_pairs takes tokens [T] and table [vocab, width]")
+    T, (vocab, width) = tokens.shape[0], table.shape
+    _need(pairs, "pairs", table.dtype)
+    if pairs.dim() != 2 or pairs.shape[1] != width or pairs.shape[0] < 2:
+        raise KernelError(f"pairs has shape {tuple(pairs.shape)}, expected [buckets + 1, {width}]")
+    if not 0 <= int(mul_prev) < 2 ** 31 or not 0 <= int(mul_cur) < 2 ** 31:
+        raise KernelError(f"factors {mul_prev} and {mul_cur} must be within 0 .. 2^31 - 1")
+    _need(positions, "positions", torch.int32, (T,))
+    _need(token_seq, "token_seq", torch.int32, (T,))
+    S = slot_id.numel()
+    _need(slot_id, "slot_id", torch.int32, (S,))
+    _need(seq_start, "seq_start", torch.int32, (S + 1,))
+    if not state.is_cuda or state.dtype != torch.int32 or state.dim() != 2 or state.shape[1] != 1:
+        raise KernelError(f"state must be int32 [slots, 1] on the GPU, got {state.dtype} "
+                          f"{tuple(state.shape)}")
+    out = torch.empty((T, width), dtype=torch.float32, device=table.device)
+    copy = None if copy_dtype is None else torch.empty((T, width), dtype=copy_dtype,
+                                                       device=table.device)
+    rc = _fn("norm", "za_embed_pairs")(
+        _ptr(tokens), _ptr(table), _ptr(pairs), _code(table.dtype), _ptr(positions), _ptr(token_seq),
+        _ptr(seq_start), _ptr(slot_id), state.data_ptr(), max(1, state.stride(0)),
+        pairs.shape[0] - 1, int(mul_prev), int(mul_cur), _ptr(out), _ptr(copy),
+        _code(copy_dtype or torch.float32), T, width, vocab, _stream())
+    _check(rc, "embed_pairs")
+    return out, copy
 
 
 def add_layernorm(residual: Optional[torch.Tensor], delta: Optional[torch.Tensor],
@@ -1656,17 +1709,23 @@ def scaled_add_rmsnorm(residual: torch.Tensor, a: torch.Tensor, scale_a: float,
     return out
 
 
-def clamped_glu(gate_up: torch.Tensor, limit: float, alpha: float, up_offset: float) -> torch.Tensor:
+def clamped_glu(gate_up: torch.Tensor, limit: float, alpha: float, up_offset: float,
+                row_scale: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``g * sigmoid(alpha * g) * (u + up_offset)`` with ``g = min(gate, limit)`` and
-    ``u = clamp(up, -limit, limit)`` on ``gate_up [T, 2I]``; ``limit <= 0``: unbounded."""
+    ``u = clamp(up, -limit, limit)`` on ``gate_up [T, 2I]``; ``limit <= 0``: unbounded.  With
+    ``row_scale`` (32-bit, one number a row) ``gate`` and ``up`` are multiplied by it first."""
     _need(gate_up, "gate_up", (torch.float32, torch.bfloat16))
     if gate_up.dim() != 2 or gate_up.shape[1] % 2:
         raise KernelError(f"clamped_glu takes [T, 2I], got {tuple(gate_up.shape)}")
     T, two_i = gate_up.shape
+    if row_scale is not None:
+        _need(row_scale, "row_scale", torch.float32)
+        if row_scale.numel() != T:
+            raise KernelError(f"row_scale holds {row_scale.numel()} numbers for {T} rows")
     out = torch.empty((T, two_i // 2), dtype=gate_up.dtype, device=gate_up.device)
-    rc = _fn("activation", "za_clamped_glu")(_ptr(gate_up), _ptr(out), _code(gate_up.dtype), T,
-                                             two_i // 2, float(limit), float(alpha),
-                                             float(up_offset), _stream())
+    rc = _fn("activation", "za_clamped_glu")(_ptr(gate_up), _ptr(out), _code(gate_up.dtype),
+                                             _ptr(row_scale), T, two_i // 2, float(limit),
+                                             float(alpha), float(up_offset), _stream())
     _check(rc, "clamped_glu")
     return out
 
@@ -2061,6 +2120,98 @@ def retention_prepare(proj: torch.Tensor, q_col: int, k_col: int, v_col: int,
     return out
 
 
+def channel_decay_prepare(proj: torch.Tensor, q_col: int, k_col: int, v_col: int, low_col: int,
+                          up: torch.Tensor, bias: torch.Tensor, root: float, q_scale: float,
+                          heads: int, dk: int, dv: int) -> torch.Tensor:
+    """From an opening projection's rows ``proj [T, columns]`` (queries, keys and values of
+    ``heads`` heads at three columns, and at ``low_col`` the ``rank`` inputs of a second product
+    ``up [heads*dk, rank]``) the 32-bit vectors of the recurrence with a decay a key channel:
+    ``[T, q * q_scale | k | a | v]``, ``a = sigmoid(up low + bias)^(1 / root)``."""
+    _need(proj, "proj", (torch.float32, torch.bfloat16))
+    if proj.dim() != 2 or up.dim() != 2:
+        raise KernelError(f"proj must be [T, columns] and up [channels, rank], got "
+                          f"{tuple(proj.shape)} and {tuple(up.shape)}")
+    T, stride = proj.shape
+    hk, hv, rank = heads * dk, heads * dv, up.shape[1]
+    _need(up, "up", (torch.float32, torch.bfloat16), (hk, rank))
+    _need(bias, "bias", torch.float32, (hk,))
+    for name, col, n in (("q_col", q_col, hk), ("k_col", k_col, hk), ("v_col", v_col, hv),
+                         ("low_col", low_col, rank)):
+        if col < 0 or col + n > stride:
+            raise KernelError(f"{name}: columns {col}..{col + n} of {stride}")
+    if not root > 0.0:
+        raise KernelError(f"the root of the decays must be positive, got {root}")
+    width = -(-(3 * hk + hv) // 4) * 4
+    out = torch.empty((T, width), dtype=torch.float32, device=proj.device)
+    rc = _fn("recurrent", "za_channel_decay_prepare")(
+        _ptr(proj), _code(proj.dtype), stride, int(q_col), int(k_col), int(v_col), int(low_col), rank,
+        _ptr(up), _code(up.dtype), _ptr(bias), float(root), float(q_scale), _ptr(out), width, T,
+        heads, dk, dv, _stream())
+    _check(rc, "channel_decay_prepare")
+    return out
+
+
+def _channel_shapes(vectors, state, state_offset, slot_id, heads, dk, dv):
+    _need(vectors, "vectors", torch.float32)
+    if vectors.dim() != 2 or vectors.shape[1] < heads * (3 * dk + dv):
+        raise KernelError(f"vectors has shape {tuple(vectors.shape)}, expected [T, >= "
+                          f"{heads * (3 * dk + dv)}]")
+    _need(slot_id, "slot_id", torch.int32, (slot_id.numel(),))
+    base, slot_stride = _state_window(state, state_offset, heads * dk * dv, "state")
+    return base, slot_stride, recurrence_plan(dk, dv)[0]
+
+
+def channel_recurrence(vectors: torch.Tensor, state: torch.Tensor, state_offset: int,
+                       seq_start: torch.Tensor, slot_id: torch.Tensor, heads: int, dk: int,
+                       dv: int) -> torch.Tensor:
+    """``S <- diag(a) S + k v^T;  o = S^T q`` token by token, a decay a head and key channel:
+    ``vectors`` as ``channel_decay_prepare`` leaves them, the state of slot ``s`` at ``state[s,
+    state_offset:]`` as ``[heads][dv][dk]``.  Returns 32-bit ``[T, heads*dv]``."""
+    base, slot_stride, lanes = _channel_shapes(vectors, state, state_offset, slot_id, heads, dk, dv)
+    T, S = vectors.shape[0], slot_id.numel()
+    _need(seq_start, "seq_start", torch.int32, (S + 1,))
+    out = torch.empty((T, heads * dv), dtype=torch.float32, device=vectors.device)
+    rc = _fn("recurrent", "za_channel_recurrence")(
+        _ptr(vectors), vectors.shape[1], base, slot_stride, _ptr(seq_start), _ptr(slot_id), _ptr(out),
+        T, S, heads, dk, dv, lanes, _stream())
+    _check(rc, "channel_recurrence", f"heads={heads} dk={dk} dv={dv}")
+    return out
+
+
+CHANNEL_CHUNK = 256            # rows of a work item of the chunked walk with channel decays
+
+
+def channel_recurrence_chunked(vectors: torch.Tensor, state: torch.Tensor, state_offset: int,
+                               slot_id: torch.Tensor, items, heads: int, dk: int,
+                               dv: int) -> torch.Tensor:
+    """``channel_recurrence`` for steps with long portions: ``items``
+    (``StepContext.attention_items(CHANNEL_CHUNK)``) cut every request's rows into chunks that
+    are walked side by side from empty states; the states before each chunk follow from a short
+    pass over the chunks, and what they add to each token's read-out is added afterwards
+    (csrc/recurrent.hip).  ``vectors`` is used up (its queries are overwritten).  Same result as
+    the plain walk up to the order of 32-bit operations."""
+    item_seq, item_row0, item_count, n_items = items
+    base, slot_stride, lanes = _channel_shapes(vectors, state, state_offset, slot_id, heads, dk, dv)
+    T, S = vectors.shape[0], slot_id.numel()
+    for name, t in (("item_seq", item_seq), ("item_row0", item_row0), ("item_count", item_count)):
+        _need(t, name, torch.int32)
+        if t.numel() < n_items:
+            raise KernelError(f"{name} holds {t.numel()} entries, fewer than {n_items} items")
+    if n_items < S:
+        raise KernelError(f"{n_items} items for {S} requests")
+    dev = vectors.device
+    out = torch.empty((T, heads * dv), dtype=torch.float32, device=dev)
+    chunk_state = torch.zeros((n_items, heads * dv * dk), dtype=torch.float32, device=dev)
+    total = torch.empty((n_items, heads * dk), dtype=torch.float32, device=dev)
+    iota = torch.arange(n_items, dtype=torch.int32, device=dev)
+    rc = _fn("recurrent", "za_channel_recurrence_chunked")(
+        _ptr(vectors), vectors.shape[1], base, slot_stride, _ptr(slot_id), _ptr(item_seq),
+        _ptr(item_row0), _ptr(item_count), _ptr(iota), n_items, S, CHANNEL_CHUNK, _ptr(chunk_state),
+        _ptr(total), _ptr(out), T, heads, dk, dv, lanes, _stream())
+    _check(rc, "channel_recurrence_chunked", f"heads={heads} dk={dk} dv={dv} items={n_items}")
+    return out
+
+
 def gated_group_norm(y: torch.Tensor, gate: torch.Tensor, gate_col: int, weight: torch.Tensor,
                      group: int, eps: float, activation: str, gate_first: bool,
                      out_scale: float = 1.0) -> torch.Tensor:
@@ -2182,10 +2333,12 @@ def route_topk(logits: torch.Tensor, n: int, top: int, correction: Optional[torc
 
 def experts_combine(expert_out: Optional[torch.Tensor], chosen: torch.Tensor, weight: torch.Tensor,
                     x: torch.Tensor, n_real: int, shared: Optional[torch.Tensor] = None,
-                    gate_logits: Optional[torch.Tensor] = None, gate_col: int = 0) -> torch.Tensor:
+                    gate_logits: Optional[torch.Tensor] = None, gate_col: int = 0,
+                    weigh: bool = True) -> torch.Tensor:
     """``y[t] = sum_j weight[t, j] * (expert_out[t * top + j] if chosen[t, j] < n_real else
     x[t]) + gate(t) * shared[t]`` as 32-bit ``[T, width]``; ``gate(t)`` is
-    ``sigmoid(gate_logits[t, gate_col])`` (32-bit logits) or one."""
+    ``sigmoid(gate_logits[t, gate_col])`` (32-bit logits) or one.  ``weigh`` false: the rows of
+    ``expert_out`` hold their weights already."""
     T, top = chosen.shape
     _need(chosen, "chosen", torch.int32, (T, top))
     _need(weight, "weight", torch.float32, (T, top))
@@ -2213,7 +2366,7 @@ def experts_combine(expert_out: Optional[torch.Tensor], chosen: torch.Tensor, we
     rc = _fn("experts", "za_experts_combine")(
         _ptr(expert_out), _code(dtype or torch.float32), _ptr(chosen), _ptr(weight), _ptr(x),
         _code(x.dtype), _ptr(shared), gate_ptr, gate_ld, _ptr(y), T, top, int(n_real), width,
-        _stream())
+        1 if weigh else 0, _stream())
     _check(rc, "experts_combine")
     return y
 
@@ -2249,16 +2402,26 @@ def table_gate(g: torch.Tensor, ids: torch.Tensor, table: torch.Tensor, col0: in
 
 
 def normed_add_(stream: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float,
-                scale: float = 1.0) -> torch.Tensor:
-    """``stream += scale * y / sqrt(mean(y^2) + eps) * weight`` in 32-bit, in place."""
+                scale: float = 1.0, copy_dtype: Optional[torch.dtype] = None):
+    """``stream += scale * y / sqrt(mean(y^2) + eps) * weight`` in 32-bit, in place; ``y [T,
+    width]`` or a stack ``[P, T, width]`` of 32-bit partial sums.  With ``copy_dtype`` the sum
+    rounded to that type comes back, otherwise the stream itself."""
     n, width = stream.shape
     _need(stream, "stream", torch.float32, (n, width))
-    _need(y, "y", (torch.float32, torch.bfloat16), (n, width))
+    partials, stride = 1, 0
+    if y.dim() == 3:
+        partials, stride = y.shape[0], n * width
+        _need(y, "y", torch.float32, (partials, n, width))
+    else:
+        _need(y, "y", (torch.float32, torch.bfloat16), (n, width))
     _need(weight, "weight", torch.float32, (width,))
-    rc = _fn("norm", "za_normed_add")(_ptr(stream), _ptr(y), _code(y.dtype), _ptr(weight), n, width,
-                                      float(eps), float(scale), _stream())
+    copy = None if copy_dtype is None else torch.empty((n, width), dtype=copy_dtype,
+                                                       device=stream.device)
+    rc = _fn("norm", "za_normed_add")(
+        _ptr(stream), _ptr(y), _code(y.dtype), partials, stride, _ptr(weight), _ptr(copy),
+        _code(copy_dtype or torch.float32), n, width, float(eps), float(scale), _stream())
     _check(rc, "normed_add_")
-    return stream
+    return stream if copy is None else copy
 
 
 # ------------------------------------------------------------ latent attention
@@ -2282,19 +2445,23 @@ def _latent_plane(plane: torch.Tensor, dtype, width: int) -> Tuple[int, int]:
 
 
 def latent_prepare(down: torch.Tensor, q_col: int, q_rank: int, c_col: int, kv_rank: int,
-                   rot_dim: int, q_norm_w: torch.Tensor, c_norm_w: torch.Tensor, eps: float,
-                   positions: torch.Tensor, slots: Optional[torch.Tensor],
+                   rot_dim: int, q_norm_w: torch.Tensor, c_norm_w: Optional[torch.Tensor],
+                   eps: float, positions: torch.Tensor, slots: Optional[torch.Tensor],
                    inv_freq: Optional[torch.Tensor], rot_dims: int, adjacent_pairs: bool,
-                   plane: Optional[torch.Tensor]) -> torch.Tensor:
+                   plane: Optional[torch.Tensor], magnitude: float = 1.0) -> torch.Tensor:
     """From the rows of a latent attention's opening projection ``down [T, columns]``: the
     RMS-normed query latent ``[T, q_rank]`` (returned), and, with ``plane``, each token's
-    cached row ``[rmsnorm(latent) | rotated key part]`` written to its place ``slots[t]``."""
+    cached row ``[rmsnorm(latent) | rotated key part]`` written to its place ``slots[t]``
+    (without ``plane`` the rows need not hold a latent).  ``magnitude``: a factor on cosine and
+    sine."""
     _need(down, "down", (torch.float32, torch.bfloat16))
     T, ld = down.shape
     _need(q_norm_w, "q_norm_w", torch.float32, (q_rank,))
-    _need(c_norm_w, "c_norm_w", torch.float32, (kv_rank,))
+    if plane is not None:
+        _need(c_norm_w, "c_norm_w", torch.float32, (kv_rank,))
     _need(positions, "positions", torch.int32, (T,))
-    if q_col < 0 or q_col + q_rank > ld or c_col < 0 or c_col + kv_rank + rot_dim > ld:
+    if q_col < 0 or q_col + q_rank > ld or c_col < 0 \
+            or (plane is not None and c_col + kv_rank + rot_dim > ld):
         raise KernelError(f"the projection's rows hold {ld} elements")
     if rot_dims % 2 or not 0 <= rot_dims <= rot_dim:
         raise KernelError(f"rot_dims {rot_dims} must be even and at most {rot_dim}")
@@ -2307,19 +2474,20 @@ def latent_prepare(down: torch.Tensor, q_col: int, q_rank: int, c_col: int, kv_r
     cq = torch.empty((T, q_rank), dtype=down.dtype, device=down.device)
     rc = _fn("latent", "za_latent_prepare")(
         _ptr(down), _code(down.dtype), ld, int(q_col), int(q_rank), int(c_col), int(kv_rank),
-        int(rot_dim), _ptr(q_norm_w), _ptr(c_norm_w), float(eps), _ptr(positions),
+        int(rot_dim), _ptr(q_norm_w), _ptr(c_norm_w) if plane is not None else None, float(eps),
+        _ptr(positions),
         _ptr(slots) if plane is not None else None, _ptr(inv_freq) if rot_dims else None,
-        int(rot_dims), 1 if adjacent_pairs else 0, _ptr(cq), _ptr(plane), page_size, stride, T,
-        _stream())
+        int(rot_dims), 1 if adjacent_pairs else 0, float(magnitude), _ptr(cq), _ptr(plane),
+        page_size, stride, T, _stream())
     _check(rc, "latent_prepare")
     return cq
 
 
 def rotate_part_(src: torch.Tensor, src_col: int, dst: torch.Tensor, dst_col: int, rot_dim: int,
                  positions: torch.Tensor, inv_freq: Optional[torch.Tensor], rot_dims: int,
-                 adjacent_pairs: bool) -> torch.Tensor:
+                 adjacent_pairs: bool, magnitude: float = 1.0) -> torch.Tensor:
     """``dst[t, h, dst_col : dst_col + rot_dim]`` takes ``src[t, h, src_col : ...]`` with its
-    first ``rot_dims`` elements rotated by the token's position."""
+    first ``rot_dims`` elements rotated by the token's position, times ``magnitude``."""
     _need(src, "src", (torch.float32, torch.bfloat16))
     _need(dst, "dst", src.dtype)
     if src.dim() != 3 or dst.dim() != 3 or src.shape[:2] != dst.shape[:2]:
@@ -2335,7 +2503,7 @@ def rotate_part_(src: torch.Tensor, src_col: int, dst: torch.Tensor, dst_col: in
     rc = _fn("latent", "za_rotate_part")(
         _ptr(src), _code(src.dtype), src.shape[2], int(src_col), _ptr(dst), dst.shape[2],
         int(dst_col), T, H, int(rot_dim), _ptr(positions), _ptr(inv_freq) if rot_dims else None,
-        int(rot_dims), 1 if adjacent_pairs else 0, _stream())
+        int(rot_dims), 1 if adjacent_pairs else 0, float(magnitude), _stream())
     _check(rc, "rotate_part_")
     return dst
 

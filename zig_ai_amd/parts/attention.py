@@ -289,7 +289,7 @@ class GroupedQueryAttention(Mixer):
         pos = params.get("position")
         self.position = None
         if pos is not None:
-            self.position = lookup("position", pos.kind)(pos.params, {}, runtime)
+            self.position = lookup("position", pos.kind)(pos.params, {}, runtime).without_magnitude()
         self.fused_rotation = bool(getattr(self.position, "fused_rotation", False))
         # recorded into a graph only if the position encoding, too, never looks at a
         # step's numbers on the host

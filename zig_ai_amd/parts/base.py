@@ -15,7 +15,8 @@ never learns which model it is in.  Five families exist:
   arrangement        wires a block's parts (it declares their names and families;
                      two norms, a mixer and a feed-forward in the usual block)
 
-plus the embedding and the output head.  All ``forward`` functions take packed
+plus the embedding (``forward(token_ids)``; one that declares a cache need,
+``forward(token_ids, step, cache)``) and the output head.  All ``forward`` functions take packed
 token rows ``[T, width]``: the tokens of every request in the step, one after
 the other; ``step`` says where each request's rows begin and what it has cached.
 """
@@ -158,6 +159,9 @@ class Mixer(Part):
     # run reads its rows when the first projection runs): a part must be done with ``x``
     # before it adds anything to ``stream``, or the norm would see the sum.
     takes_stream = False
+    # An arrangement whose next kernel adds up stacks of partial sums sets this on the part;
+    # a part that knows it may then return one (``[P, T, width]``, 32-bit).
+    partial_ok = False
 
     @classmethod
     def cache_need(cls, params: Mapping[str, Any]):
@@ -170,6 +174,7 @@ class Mixer(Part):
 
 class FeedForward(Part):
     takes_stream = False      # as for Mixer
+    partial_ok = False        # as for Mixer
     opens_with_swiglu = False  # its first product is ``ops.linear_swiglu`` on what it is handed
 
     def forward(self, x: torch.Tensor, step) -> torch.Tensor:
@@ -214,6 +219,13 @@ class PositionEncoding(Part):
     # ``kernel_sources`` and ``item_granularities``.  ``graph_safe = True`` only if
     # ``apply`` never looks at ``positions`` (or anything of the step) on the host.
     graph_safe = False
+    magnitude = 1.0    # factor on what is rotated, besides the rotation
+
+    def without_magnitude(self) -> "PositionEncoding":
+        """This encoding, for a mixer whose kernels rotate without such a factor."""
+        if self.magnitude != 1.0:
+            raise ValueError("this mixer's kernels rotate without a factor on cosine and sine")
+        return self
 
     def apply(self, q: torch.Tensor, k: torch.Tensor, positions: torch.Tensor):
         """Generic path: return encoded ``(q, k)`` of shape ``[T, heads, head_dim]``."""

@@ -133,6 +133,80 @@ register_arrangement(ParallelResidualBlock.kind, ParallelResidualBlock)
 register_arrangement(ParallelMixerBlock.kind, ParallelMixerBlock)
 
 
+class NormedOutputBlock:
+    """Norms on the parts' outputs only; the parts read the stream itself:
+
+        h = x + norm1(mixer(x));   y = h + norm2(feed_forward(h))
+
+    One kernel adds a part's result up (it may be a stack of partial sums), norms it, adds it
+    to the 32-bit stream and leaves the sum rounded for the part that follows, also across
+    the boundary between two blocks (``step.rounded``); nothing is left pending."""
+
+    kind = "normed_output"
+    slots = {"mixer": "mixer", "mixer_norm": "norm", "feed_forward": "feed_forward",
+             "feed_forward_norm": "norm"}
+    leaves_rounded = True
+
+    def __init__(self, parts):
+        self.parts = dict(parts)
+        self.mixer, self.mixer_norm = parts["mixer"], parts["mixer_norm"]
+        self.feed_forward = parts.get("feed_forward")
+        self.feed_forward_norm = parts.get("feed_forward_norm")
+        for part in (self.mixer, self.feed_forward):
+            if part is not None and hasattr(part, "partial_ok"):
+                part.partial_ok = True
+
+    def forward(self, residual: torch.Tensor, pending: Optional[torch.Tensor], step,
+                cache) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
+        from ..kernels import ops
+        if pending is not None:
+            ops.stream_add_(residual, pending)
+            step.rounded = None
+        self._add(residual, self.mixer_norm, self.mixer.forward(self._input(residual, step), step,
+                                                                cache), step)
+        if self.feed_forward is not None:
+            self._add(residual, self.feed_forward_norm,
+                      self.feed_forward.forward(self._input(residual, step), step), step)
+        return residual, None
+
+    def _dtype(self) -> torch.dtype:
+        runtime = getattr(self.mixer, "runtime", None)
+        return runtime.dtype if runtime is not None else torch.float32
+
+    def _input(self, residual: torch.Tensor, step) -> torch.Tensor:
+        """What a part reads: the stream, rounded to the run's type."""
+        from ..kernels import ops
+        dtype = self._dtype()
+        if dtype == torch.float32:
+            return residual
+        x, step.rounded = step.rounded, None
+        return x if x is not None else ops.cast(residual, dtype)
+
+    def _add(self, residual: torch.Tensor, norm, y: torch.Tensor, step) -> None:
+        from ..kernels import ops
+        dtype = self._dtype()
+        if hasattr(norm, "weight") and hasattr(norm, "eps") and not hasattr(norm, "bias"):
+            copy = ops.normed_add_(residual, y, norm.weight, norm.eps,
+                                   copy_dtype=None if dtype == torch.float32 else dtype)
+            step.rounded = copy if copy is not residual else None
+            return
+        if y.dim() == 3:
+            y = y.sum(dim=0)
+        ops.stream_add_(residual, norm.forward(y))
+        step.rounded = None
+
+
+class NormedOutputMixerBlock(NormedOutputBlock):
+    """The same for a layer that has no feed-forward: ``y = x + norm1(mixer(x))``."""
+
+    kind = "normed_output_no_ff"
+    slots = {"mixer": "mixer", "mixer_norm": "norm"}
+
+
+register_arrangement(NormedOutputBlock.kind, NormedOutputBlock)
+register_arrangement(NormedOutputMixerBlock.kind, NormedOutputMixerBlock)
+
+
 class ScaledResidualBlock:
     """A pre-norm block whose parts enter the stream with weights, and which may run two
     mixers side by side on the same normed input and may lack the feed-forward:

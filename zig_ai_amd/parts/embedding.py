@@ -4,9 +4,12 @@ head (a projection to 32-bit logits, optionally sharing the embedding table).
 id outside the table is an error raised before the launch) and
 /root/reference/src/loader/gguf_model.zig:47-54 (tied fallback).
 
-Two options for designs that need them: ``token_embedding`` with ``norm`` (the rows that
-open the stream are RMS-normed, ``x / sqrt(mean(x^2) + norm_eps) * norm.weight``, in 32-bit)
-and ``linear_head`` with ``softcap`` (``logits <- softcap * tanh(logits / softcap)``)."""
+Options for designs that need them: ``token_embedding`` with ``norm`` (the rows that
+open the stream are RMS-normed, ``x / sqrt(mean(x^2) + norm_eps) * norm.weight``, in 32-bit);
+with ``pair = {buckets, mul_prev, mul_cur}`` (a second table of ``buckets + 1`` rows adds the row
+``(token before * mul_prev + token * mul_cur) mod buckets``, for a request's first token the last
+row; a request's last token is state, kept in its slot); ``linear_head`` with ``softcap``
+(``logits <- softcap * tanh(logits / softcap)``)."""
 
 from __future__ import annotations
 
@@ -15,7 +18,7 @@ from typing import Any, Dict, Mapping
 import torch
 
 from ..kernels import ops
-from .base import Part, Runtime, TensorRule, register_embedding, register_head
+from .base import Part, Runtime, StateNeed, TensorRule, register_embedding, register_head
 
 
 class TokenEmbedding(Part):
@@ -29,7 +32,15 @@ class TokenEmbedding(Part):
                                       role="table")}
         if params.get("norm"):
             rules["norm.weight"] = TensorRule(((int(params["hidden_size"]),),), role="norm")
+        if params.get("pair"):
+            rules["pair.weight"] = TensorRule(((int(params["pair"]["buckets"]) + 1,
+                                                int(params["hidden_size"])),), role="table")
         return rules
+
+    @classmethod
+    def cache_need(cls, params: Mapping[str, Any]):
+        """With ``pair``: the request's last token."""
+        return StateNeed((1,), torch.int32) if params.get("pair") else None
 
     def __init__(self, params, tensors, runtime: Runtime):
         super().__init__(params, tensors, runtime)
@@ -38,9 +49,22 @@ class TokenEmbedding(Part):
         # a norm on the rows that open the stream (None: none)
         self.norm_weight = tensors["norm.weight"] if params.get("norm") else None
         self.norm_eps = float(params.get("norm_eps", 0.0))
+        self.pair = dict(params["pair"]) if params.get("pair") else None
+        if self.pair is not None:
+            self.pair_weight = tensors["pair.weight"]
+            if self.pair_weight.dtype != self.weight.dtype:
+                self.weight, self.pair_weight = self.weight.float(), self.pair_weight.float()
 
-    def forward(self, token_ids: torch.Tensor) -> torch.Tensor:
-        x = ops.embed_gather(token_ids, self.weight)
+    def forward(self, token_ids: torch.Tensor, step=None, cache=None) -> torch.Tensor:
+        if self.pair is not None:
+            rounded = self.runtime.dtype if self.runtime.dtype != torch.float32 \
+                and self.norm_weight is None else None
+            x, step.rounded = ops.embed_pairs(
+                token_ids, self.weight, self.pair_weight, step.positions, step.token_seq,
+                step.seq_start, step.slot_id, cache.state, self.pair["mul_prev"],
+                self.pair["mul_cur"], rounded)
+        else:
+            x = ops.embed_gather(token_ids, self.weight)
         if self.norm_weight is not None:
             x = ops.add_rmsnorm(x, None, self.norm_weight, self.norm_eps, torch.float32,
                                 write_residual=False)
@@ -72,7 +96,7 @@ class LinearHead(Part):
             raise ValueError(f"the logits' cap must not be negative, got {self.softcap}")
 
     def forward(self, x) -> torch.Tensor:
-        if not self.tied and self.weight.dtype == torch.bfloat16 and self.weight.shape[1] % 8:
+        if self.weight.dtype == torch.bfloat16 and self.weight.shape[1] % 8:
             self.weight = ops.projection_weight(self.weight)     # kept in 32-bit from now on
         ops.check_projection_weight(self.weight, "output head")
         logits = ops.linear(x, self.weight, out_dtype=torch.float32, tune=self.runtime.tune)

@@ -92,12 +92,18 @@ class RoutedExperts(FeedForward):
         neighbouring outputs (a group counts by its largest choice score; ``groups = 0``: no
         limit); weight = s * route_scale (``renormalize``: divided by the chosen scores' sum)
         y = sum_chosen weight_e * expert_e(x) + gate * shared(x)
+                                       (``weight_on="input"``: expert_e(weight_e * x))
 
-    ``expert_e(x) = Wdown_e (act(Wgate_e x) * (Wup_e x))`` for the ``experts`` outputs that have
+    ``expert_e(x) = Wdown_e (act(Wgate_e x) * (Wup_e x))``, or with ``activation="bounded_glu"``
+    ``Wdown_e (g * sigmoid(gate_slope * g) * (u + up_offset))`` with ``g = min(Wgate_e x, bound)``,
+    ``u = clamp(Wup_e x, -bound, bound)``, for the ``experts`` outputs that have
     weights; the ``identity_experts`` outputs behind them hand ``x`` on.  ``shared_size > 0``:
     one more expert of that width runs for every token, times ``sigmoid(Wsg x)`` (one number
     a token) when ``shared_gate``.  The router's product and everything after it up to the
-    weights is 32-bit; the weighted sum is taken in 32-bit in a fixed order.
+    weights is 32-bit; the weighted sum is taken in 32-bit in a fixed order.  A
+    weight on the input is applied to the gate|up product (the same numbers: there are no
+    biases) in front of the bounds; the experts' results then add up without weights, as a
+    stack of partial sums where the arrangement takes one (``partial_ok``).
 
     Nothing is looked at on the host: the router's choice becomes per-expert lists on the
     device and two grouped products run every expert's rows in one launch each."""
@@ -150,9 +156,19 @@ class RoutedExperts(FeedForward):
         self.scores = str(params.get("scores", "softmax"))
         self.renormalize = bool(params.get("renormalize", False))
         self.activation = str(params.get("activation", "silu"))
-        if self.activation not in ops.GATE_ACTIVATIONS:
-            raise ValueError(f"expert activation must be one of {sorted(ops.GATE_ACTIVATIONS)}, "
-                             f"got {self.activation!r}")
+        if self.activation not in ops.GATE_ACTIVATIONS and self.activation != "bounded_glu":
+            raise ValueError(f"expert activation must be bounded_glu or one of "
+                             f"{sorted(ops.GATE_ACTIVATIONS)}, got {self.activation!r}")
+        if self.activation == "bounded_glu":
+            self.bound, self.slope, self.offset = (float(params[k]) for k in
+                                                   ("bound", "gate_slope", "up_offset"))
+        self.weight_on = str(params.get("weight_on", "output"))
+        if self.weight_on not in ("input", "output"):
+            raise ValueError(f"weight_on must be input or output, got {self.weight_on!r}")
+        if self.weight_on == "input" and self.activation != "bounded_glu":
+            raise ValueError("a weight on the experts' input is applied by the bounded gate only")
+        if S and self.activation == "bounded_glu":
+            raise ValueError("a shared expert takes one of the plain gate activations")
         self.correction = tensors["correction"] if params.get("correction") else None
         # the router's rows and, behind them, the shared expert's gate: one 32-bit product
         rows = [tensors["router.weight"]]
@@ -189,9 +205,18 @@ class RoutedExperts(FeedForward):
             lists, counts = ops.expert_lists(None, chosen, T, self.experts)
             a = ops.grouped_linear(x, self.gate_up, lists, counts, T, per_token=True,
                                    out_dtype=x.dtype)
-            a = ops.gated_unit(a, self.activation)
+            if self.activation == "bounded_glu":
+                a = ops.clamped_glu(a, self.bound, self.slope, self.offset,
+                                    weight if self.weight_on == "input" else None)
+            else:
+                a = ops.gated_unit(a, self.activation)
+            # (nothing but the experts' own results to add up: left to the next kernel)
+            stacked = self.partial_ok and self.weight_on == "input" and not self.identity \
+                and self.shared_gate_up is None
             out = ops.grouped_linear(a, self.down, lists, counts, T, per_token=False,
-                                     out_dtype=torch.float32)
+                                     stacked=stacked, out_dtype=torch.float32)
+            if stacked:
+                return out
         shared = None
         if self.shared_gate_up is not None:
             if x.dtype == torch.bfloat16 and self.shared_gate_up.dtype == torch.bfloat16 \
@@ -202,7 +227,8 @@ class RoutedExperts(FeedForward):
                 s = ops.gated_unit(ops.linear(x, self.shared_gate_up, tune=tune), self.activation)
             shared = ops.linear(s, self.shared_down, out_dtype=torch.float32, tune=tune)
         return ops.experts_combine(out, chosen, weight, x, self.experts, shared,
-                                   logits if self.shared_gated else None, self.outputs)
+                                   logits if self.shared_gated else None, self.outputs,
+                                   weigh=self.weight_on == "output")
 
 
 register_feed_forward(RoutedExperts.kind, RoutedExperts)

@@ -24,7 +24,10 @@ All sizes and constants come from ``params``: ``hidden_size, num_heads, head_dim
 rotated_dim`` (0: no positions), ``value_dim, kv_rank, q_rank, softmax_scale`` (None:
 ``(head_dim + rotated_dim)^-1/2``), ``norm_eps, sink`` (true: a tensor ``sink [num_heads]``),
 ``gate`` and ``position`` (a nested rotary spec whose ``head_dim`` is ``rotated_dim``; its
-``rotary_dim`` may be smaller: the other elements of the rotated part pass unchanged).
+``rotary_dim`` may be smaller: the other elements of the rotated part pass unchanged; its
+``magnitude`` multiplies what it turns, in queries and keys).  ``makes_rows`` (true): with false
+the layer has no ``Wdkv`` and reads the rows that another layer caches: its run-order entry
+shares that layer's cache entry (``LayerCall.cache``, ``writes_cache=False``).
 """
 
 from __future__ import annotations
@@ -77,11 +80,12 @@ class LatentAttention(Mixer):
         rules = {"q_down.weight": TensorRule(((Rq, H),)),
                  "q_norm.weight": TensorRule(((Rq,),), role="norm"),
                  "q_up.weight": TensorRule(((nh * (d + dr), Rq),)),
-                 "kv_down.weight": TensorRule(((R + dr, H),)),
-                 "kv_norm.weight": TensorRule(((R,),), role="norm"),
                  "k_up.weight": TensorRule(((nh * d, R),)),
                  "v_up.weight": TensorRule(((nh * dv, R),)),
                  "out_proj.weight": TensorRule(((H, nh * dv),))}
+        if params.get("makes_rows", True):
+            rules["kv_down.weight"] = TensorRule(((R + dr, H),))
+            rules["kv_norm.weight"] = TensorRule(((R,),), role="norm")
         if params.get("sink"):
             rules["sink"] = TensorRule(((nh,),), role="bias")
         if params.get("gate") == "head":
@@ -113,7 +117,7 @@ class LatentAttention(Mixer):
         self.sink = tensors["sink"] if params.get("sink") else None
         pos = params.get("position")
         self.position = None
-        self.rot_dims, self.adjacent, self.inv_freq = 0, False, None
+        self.rot_dims, self.adjacent, self.inv_freq, self.magnitude = 0, False, None, 1.0
         if dr:
             if pos is None:
                 raise ValueError("a rotated part needs a position encoding")
@@ -123,18 +127,22 @@ class LatentAttention(Mixer):
             self.rot_dims = self.position.rotary_dim
             self.adjacent = self.position.pairing == "adjacent"
             self.inv_freq = self.position.inv_freq
+            self.magnitude = float(self.position.magnitude)
         elif pos is not None:
             raise ValueError("a position encoding needs a rotated part")
         # the opening product: query latent | latent and rotated key part | gate, each
         # starting on a 16-byte boundary
-        pieces = [pad_rows(tensors["q_down.weight"]), pad_rows(tensors["kv_down.weight"])]
+        self.makes_rows = bool(params.get("makes_rows", True))
+        pieces = [pad_rows(tensors["q_down.weight"])]
         self.c_col = pieces[0].shape[0]
-        self.gate_col = self.c_col + pieces[1].shape[0]
+        if self.makes_rows:
+            pieces.append(pad_rows(tensors["kv_down.weight"]))
+        self.gate_col = sum(p.shape[0] for p in pieces)
         if self.gate is not None:
             pieces.append(pad_rows(tensors["gate_proj.weight"]))
         self.w_open = ops.projection_weight(fuse_rows(*pieces))
         self.q_norm = tensors["q_norm.weight"]
-        self.kv_norm = tensors["kv_norm.weight"]
+        self.kv_norm = tensors["kv_norm.weight"] if self.makes_rows else None
         self.w_q_up = ops.projection_weight(tensors["q_up.weight"])
         self.w_out = ops.projection_weight(tensors["out_proj.weight"])
         # per head: Wuk^T as [R, d] (folds into the query), Wuv as [dv, R] (expands the result)
@@ -159,18 +167,21 @@ class LatentAttention(Mixer):
         T = x.shape[0]
         tune = self.runtime.tune
         plane = cache.planes[0]
+        if cache.writes and not self.makes_rows:
+            raise ValueError("a latent attention without rows of its own reads another layer's "
+                             "cache: its run-order entry must not write")
         down = ops.linear(x, self.w_open, tune=tune)
         cq = ops.latent_prepare(down, 0, self.q_rank, self.c_col, R, dr, self.q_norm, self.kv_norm,
                                 self.eps, step.positions, step.slot_mapping[cache.group],
                                 self.inv_freq, self.rot_dims, self.adjacent,
-                                plane if cache.writes else None)
+                                plane if cache.writes else None, self.magnitude)
         q = ops.linear(cq, self.w_q_up, tune=tune).view(T, nh, d + dr)
         # the folded query [Wuk^T q_n | rot(q_r)]
         qf = torch.empty((T, nh, self.width), dtype=q.dtype, device=q.device)
         ops.head_linear(q, 0, self.k_fold, out=qf, out_col=0)
         if dr:
             ops.rotate_part_(q, d, qf, R, dr, step.positions, self.inv_freq, self.rot_dims,
-                             self.adjacent)
+                             self.adjacent, self.magnitude)
         item_seq, item_row0, item_count, n_items = step.attention_items(self.rows_per_item)
         waves = 0
         if self.mfma:
@@ -192,7 +203,7 @@ class LatentAttention(Mixer):
         if getattr(step, "taps", None) is not None:
             step.taps["q"] = qf.clone()
             step.taps["o"] = a.clone()
-        return ops.linear(a.view(T, nh * dv), self.w_out, tune=tune)
+        return ops.linear(a.view(T, nh * dv), self.w_out, partial_ok=self.partial_ok, tune=tune)
 
 
 register_mixer(LatentAttention.kind, LatentAttention)

@@ -46,6 +46,20 @@ Lightning attention is ``activation="silu"``, ``key_scale=1``, ``output_norm="al
 A step in which some request brings more than ``ops.RETENTION_CHUNK`` tokens walks its
 portions as chunks side by side (``ops.fixed_decay_recurrence_chunked``): with a constant
 decay the state is linear in what the tokens bring.
+
+``gated_linear`` (gated linear attention: a decay of its own for every key channel, made from
+the token).  Projections q, k (``num_heads x head_dim``), v and a gate g (``num_heads x
+value_dim``), no biases, no convolution, no positions; the decay is ``a = sigmoid(W_a2 W_a1 h +
+b)^(1 / decay_root)`` per head and key channel, through ``decay_rank`` numbers a token; per head
+
+    S <- diag(a) S + k v^T;   o = S^T q * head_dim^-1/2
+
+then each head's ``o`` over its root mean square (``norm_eps``), times ``norm.weight`` (one
+weight per value channel, shared by the heads), times ``silu(g)`` or ``sigmoid(g)`` (``gate``), and
+the output projection.  The second decay product, the decays, the walk and the state (in the slot)
+are 32-bit.  Long portions are walked in chunks side by side, as for ``retention``
+(``ops.channel_recurrence_chunked``): the state a chunk starts from reaches its read-outs
+through the product of the decays since, which is at most one.
 """
 
 from __future__ import annotations
@@ -262,8 +276,8 @@ class Retention(Mixer):
             raise ValueError(f"retention: activation {self.activation!r}, output_norm "
                              f"{self.output_norm!r}, gate {self.gate!r}")
         pos = params.get("position")
-        self.position = lookup("position", pos.kind)(pos.params, {}, runtime) if pos is not None \
-            else None
+        self.position = lookup("position", pos.kind)(pos.params, {}, runtime).without_magnitude() \
+            if pos is not None else None
         if self.position is not None and not (getattr(self.position, "fused_rotation", False)
                                                and self.position.pairing == "half"):
             raise ValueError("retention takes a rotary position encoding in halves, or none")
@@ -310,6 +324,80 @@ class Retention(Mixer):
         return ops.linear(h, self.w_out, accumulate=stream, tune=self.runtime.tune)
 
 
+class GatedLinearAttention(Mixer):
+    kind = "gated_linear"
+    graph_safe = True
+    takes_normed_rows = True      # ``x`` is only ever handed to ``ops.linear``
+    kernel_sources = ("gemm", "recurrent")
+
+    @staticmethod
+    def _sizes(params):
+        return tuple(int(params[k]) for k in ("hidden_size", "num_heads", "head_dim", "value_dim",
+                                              "decay_rank"))
+
+    @classmethod
+    def tensor_rules(cls, params: Mapping[str, Any]) -> Dict[str, TensorRule]:
+        W, H, d, dv, r = cls._sizes(params)
+        return {"q_proj.weight": TensorRule(((H * d, W),)),
+                "k_proj.weight": TensorRule(((H * d, W),)),
+                "v_proj.weight": TensorRule(((H * dv, W),)),
+                "gate_proj.weight": TensorRule(((H * dv, W),)),
+                "decay_down.weight": TensorRule(((r, W),)),
+                "decay_up.weight": TensorRule(((H * d, r),)),
+                "decay_up.bias": TensorRule(((H * d,),), role="bias"),
+                "norm.weight": TensorRule(((dv,),), role="norm"),
+                "out_proj.weight": TensorRule(((W, H * dv),))}
+
+    @classmethod
+    def cache_need(cls, params: Mapping[str, Any]):
+        W, H, d, dv, r = cls._sizes(params)
+        return StateNeed((H * d * dv,))
+
+    def __init__(self, params, tensors, runtime: Runtime):
+        super().__init__(params, tensors, runtime)
+        W, H, d, dv, r = self._sizes(params)
+        ops.recurrence_plan(d, dv)
+        self.heads, self.head_dim, self.value_dim = H, d, dv
+        self.eps = float(params["norm_eps"])
+        self.root = float(params["decay_root"])
+        self.gate = str(params.get("gate", "silu"))
+        if self.gate not in ("silu", "sigmoid") or not self.root > 0.0:
+            raise ValueError(f"gated_linear: gate {self.gate!r}, decay_root {self.root}")
+        # one opening product: q | k | v | g | decay_down
+        self.w_in = ops.projection_weight(pad_rows(fuse_rows(
+            tensors["q_proj.weight"], tensors["k_proj.weight"], tensors["v_proj.weight"],
+            tensors["gate_proj.weight"], tensors["decay_down.weight"])))
+        self.gate_col = 2 * H * d + H * dv
+        self.low_col = self.gate_col + H * dv
+        self.decay_up = tensors["decay_up.weight"].contiguous()
+        self.decay_bias = tensors["decay_up.bias"]
+        self.norm_w = tensors["norm.weight"]
+        self.w_out = ops.projection_weight(tensors["out_proj.weight"])
+        self.item_granularities = [ops.CHANNEL_CHUNK]
+        ops.check_projection_weight(self.w_in, "gated_linear opening projection")
+        ops.check_projection_weight(self.w_out, "gated_linear out_proj")
+
+    def forward(self, x, step, cache):
+        H, d, dv = self.heads, self.head_dim, self.value_dim
+        z = ops.linear(x, self.w_in, tune=self.runtime.tune)
+        vectors = ops.channel_decay_prepare(z, 0, H * d, 2 * H * d, self.low_col, self.decay_up,
+                                            self.decay_bias, self.root, d ** -0.5, H, d, dv)
+        if getattr(step, "taps", None) is not None:
+            step.taps["vectors"] = vectors.clone()
+        items = step.attention_items(ops.CHANNEL_CHUNK)
+        if items[3] > step.n_seqs:
+            # some request brings more than a chunk (a function of the step's shape alone)
+            o = ops.channel_recurrence_chunked(vectors, cache.state, 0, step.slot_id, items, H, d, dv)
+        else:
+            o = ops.channel_recurrence(vectors, cache.state, 0, step.seq_start, step.slot_id, H, d, dv)
+        if getattr(step, "taps", None) is not None:
+            step.taps["o"] = o.clone()
+        h = ops.gated_group_norm(o, z, self.gate_col, self.norm_w, dv, self.eps, self.gate,
+                                 gate_first=False)
+        return ops.linear(h, self.w_out, partial_ok=self.partial_ok, tune=self.runtime.tune)
+
+
 register_mixer(StateSpaceDuality.kind, StateSpaceDuality)
+register_mixer(GatedLinearAttention.kind, GatedLinearAttention)
 register_mixer(Retention.kind, Retention)
 register_mixer(GatedDeltaRule.kind, GatedDeltaRule)
