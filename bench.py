@@ -7,6 +7,7 @@
     python bench.py --workload compare --compare-design ranesun   # Ranesun beside Rudilix
     python bench.py --workload compare --compare-design gemodra   # Gemodra beside Ranesun
     python bench.py --workload compare --compare-design nopozen   # Nopozen beside Ranesun
+    python bench.py --workload compare --compare-design vupelorn  # Vupelorn beside Gemodra, Nopozen
 
 Default run: the layer sizes of the LFM2-1.2B shape (16 layers, hidden 2048, vocabulary 65,536)
 with random bfloat16 weights N(0, 0.02), a batch of 8 requests, each prefilled
@@ -46,6 +47,10 @@ the engine has (attention with sinks, experts of which a token uses a few).
 in turn, parallel blocks, dense and routed feed-forwards, the first half of the layers a looped
 span) beside a Ranesun model of the same width, depth and vocabulary, the closest design the
 engine has (a fixed-decay linear attention, attention with sinks, small experts, a loop).
+``--compare-design vupelorn``: a Vupelorn model (gated linear attention and attention over a
+cached latent in turn, routed small experts) beside a Gemodra model of the same width, depth and
+vocabulary, the closest design the engine has (the same latent attention and router), and a
+Nopozen model (whose lightning layers are the closest to gated linear attention).
 """
 
 import argparse
@@ -249,10 +254,44 @@ def nopozen_shape(width, layers, vocab):
             "max_position_embeddings": 128000}
 
 
+def vupelorn_shape(width, layers, vocab):
+    """Layer sizes in the manner of a real model of this design: gated linear attention (heads
+    of 128 x 128, decays of the sixteenth root, through 16 numbers a token) and latent attention
+    (heads of 128 unrotated and 64 rotated elements, values of 128, a latent of 512) in turn, the
+    latter with adjacent pairs or with halves and stretched frequencies in turn, every other
+    layer with adjacent pairs reading the rows of the one before it; 32 experts of half the width,
+    4 a token; a table of pairs of tokens as long as the vocabulary."""
+    heads = width // 128
+    linear = {"heads": heads, "dim": 128, "vdim": 128, "tau": 16.0, "decay_rank": 16}
+    latent = {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512,
+              "q_rank": 3 * width // 4, "scale": 192 ** -0.5, "rot": {"dims": 64, "base": 1e6}}
+    stretched = dict(latent, rot=dict(latent["rot"], scaling={"factor": 8.0, "original": 4096,
+                                                              "fast": 32.0, "slow": 1.0}))
+    mlp = {"kind": "moe", "expert": {"ff": width // 2, "limit": 7.0},
+           "router": {"experts": 32, "top": 4}}
+    out, source = [], None
+    for i in range(layers):
+        if i % 2 == 0:
+            kind, mixer = "gla", linear
+        elif i % 4 == 3:
+            kind, mixer = "latent_attention", stretched
+        else:
+            kind, mixer = "latent_attention_2", latent
+            if source is None:
+                source = i
+            else:
+                mixer, source = dict(latent, kv_from=source), None
+        out.append({"type": kind, "mixer": mixer, "mlp": mlp})
+    return {"architecture": "Vupelorn", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+            "embedding": {"bigram": {"buckets": vocab - 1, "mul_prev": 31337, "mul_cur": 17}},
+            "layers": out, "max_position_embeddings": 128000}
+
+
 def compare(widths, layers, batch, prompt_len, steps, warmup, design="rudilix", only=None) -> dict:
     """Prefill and decode throughput of Rudilix and of LFM2 at equal sizes, or
     (``design="ranesun"``) of Ranesun and of Rudilix, or (``design="gemodra"``) of Gemodra and
-    of Ranesun, or (``design="nopozen"``) of Nopozen and of Ranesun."""
+    of Ranesun, or (``design="nopozen"``) of Nopozen and of Ranesun, or
+    (``design="vupelorn"``) of Vupelorn, of Gemodra and of Nopozen."""
     import torch
     from zig_ai_amd.engine import DecoderModel, ModelRunner, StepEntry
     from zig_ai_amd.kernels import ops
@@ -341,11 +380,13 @@ def compare(widths, layers, batch, prompt_len, steps, warmup, design="rudilix", 
 
     result = {"workload": "compare", "dtype": "bf16", "data": "synthetic", "layers": layers,
               "batch": batch, "prompt_len": prompt_len, "steps": steps, "warmup": warmup, "widths": {}}
-    if design in ("ranesun", "gemodra", "nopozen"):
+    if design != "rudilix":
         for width in widths:
             pair = {"ranesun": {"ranesun": ranesun_shape, "rudilix": rudilix_shape},
                     "gemodra": {"gemodra": gemodra_shape, "ranesun": ranesun_shape},
-                    "nopozen": {"nopozen": nopozen_shape, "ranesun": ranesun_shape}}[design]
+                    "nopozen": {"nopozen": nopozen_shape, "ranesun": ranesun_shape},
+                    "vupelorn": {"vupelorn": vupelorn_shape, "gemodra": gemodra_shape,
+                                 "nopozen": nopozen_shape}}[design]
             result["widths"][str(width)] = {name: measure(shape(width, layers, vocab))
                                             for name, shape in pair.items()
                                             if only in (None, name)}
@@ -405,10 +446,10 @@ def main() -> int:
     ap.add_argument("--compare-widths", default="1024,2048",
                     help="--workload compare: the widths, with commas between them")
     ap.add_argument("--compare-layers", type=int, default=8, help="--workload compare: layers")
-    ap.add_argument("--compare-design", choices=["rudilix", "ranesun", "gemodra", "nopozen"],
+    ap.add_argument("--compare-design", choices=["rudilix", "ranesun", "gemodra", "nopozen", "vupelorn"],
                     default="rudilix",
-                    help="--workload compare: rudilix (beside LFM2), ranesun (beside Rudilix) or "
-                         "gemodra (beside Ranesun)")
+                    help="--workload compare: rudilix (beside LFM2), ranesun (beside Rudilix), "
+                         "gemodra or nopozen (beside Ranesun), vupelorn (beside Gemodra and Nopozen)")
     ap.add_argument("--compare-only", default=None,
                     help="--workload compare: measure this model of the pair alone (for a profiler)")
     ap.add_argument("--workload", choices=["steps", "serve", "compare"], default="steps",
