@@ -790,7 +790,19 @@ channel_decay_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_
     __syncthreads();
     if (c < hk) {
       const TW* w = up + (size_t)c * rank + r0;
-      for (int r = 0; r < rn; ++r) {
+      int r = 0;
+      if (rank % 8 == 0) {       // (rows of `up` start on 16-byte boundaries)
+#pragma unroll 2
+        for (; r + 8 <= rn; r += 8) {
+          float w8[8];
+          load8<TW>(w + r, w8);
+#pragma unroll
+          for (int e = 0; e < 8; ++e)
+#pragma unroll
+            for (int i = 0; i < GP_TOKENS; ++i) z[i] = fmaf(w8[e], low[i][r + e], z[i]);
+        }
+      }
+      for (; r < rn; ++r) {
         const float wv = to_f32<TW>(w[r]);
 #pragma unroll
         for (int i = 0; i < GP_TOKENS; ++i) z[i] = fmaf(wv, low[i][r], z[i]);
@@ -838,7 +850,265 @@ extern "C" int za_channel_decay_prepare(const void* proj, int dtype, int proj_st
   return za_launch_status();
 }
 
-// The plain walk with these vectors (`vectors` as channel_decay_prepare leaves them).
+// Portions of many tokens: blocks of up to CM_TOKENS tokens at a time, as matrix products on the
+// matrix cores in their 32-bit form (v_mfma_f32_16x16x4_f32: products and sums in full
+// 32-bit).  Within a block that starts from state S, with a_1 its first token's decays and
+// L_i = a_2 ... a_i (per channel, L_1 = 1; S' = diag(a_1) S):
+//     o_i = S'^T (q_i L_i) + sum_(j <= i) ((q_i L_i) . (k_j / L_j)) v_j
+//     S  <- diag(L_n) (S' + sum_j (k_j / L_j) v_j^T)
+// A block ends before a token that would take any channel's L below CM_FLOOR, so that k / L stays
+// finite and every sum keeps the precision of its largest term; the token then opens the next
+// block, where its own decays only multiply the state: decays may be as small as they like,
+// zero included, and only make blocks shorter.
+// A workgroup serves 64 columns of one walker's head, 16 a wave: a wave keeps its columns'
+// state in accumulators, whose layout (rows 4 g + i of a tile in register i of lane group g)
+// is that of the second operand when k runs as 4 g + j, so S enters q S and leaves K^T V
+// without moving.  What a token brings is requested one block ahead.
+#define CM_TOKENS 16
+#define CM_FLOOR 7.8886090522101181e-31f     // 2^-100
+#define CM_LD (CM_TOKENS + 4)                // padded row of 16 tokens, 16-byte aligned
+
+struct ChannelArgs {
+  const float* vectors;    // [T][width]: q | k | decays | v
+  int width;
+  float* state;            // per slot [H][dv][dk]
+  long long slot_stride;
+  const int* start;        // first row of walker w
+  const int* count;        // its rows, or null: start[w + 1] - start[w]
+  const int* slot_id;      // null: walker w uses slot w, and starts from an empty state
+  float* out;              // [T][H*dv]
+  float* scaled_q;         // null, or [T][H*dk]: q times all decays since the walker's start
+  float* total;            // null, or [walkers][H*dk]: the product of all its decays
+  int H, dk, dv;
+};
+
+template <int NT>     // tiles of 16 key channels
+__global__ void __launch_bounds__(256)
+channel_blocks_kernel(ChannelArgs a) {
+  constexpr int DK = NT * 16, QLD = DK + 4;
+  constexpr int UNITS = 2 * DK;                       // (q or k) x channel
+  constexpr int U = UNITS <= 256 ? 1 : UNITS / 256;   // units a thread
+  __shared__ __attribute__((aligned(16))) float qs[CM_TOKENS][QLD];     // q L
+  __shared__ __attribute__((aligned(16))) float ks[CM_TOKENS][QLD];     // k / L
+  __shared__ __attribute__((aligned(16))) float kt[DK][CM_LD];          // the same, turned round
+  __shared__ __attribute__((aligned(16))) float part[4][16][CM_LD];     // q L . k / L, by range of k
+  __shared__ __attribute__((aligned(16))) float grow[DK];               // the state's next factor
+  __shared__ int shortest;
+
+  const int w = blockIdx.x, h = blockIdx.y;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int r16 = lane & 15, g = lane >> 4;
+  const int dk = a.dk, dv = a.dv, hk = a.H * dk;
+  const int row0 = a.start[w], n_rows = a.count ? a.count[w] : a.start[w + 1] - row0;
+  const int col = blockIdx.z * 64 + wave * 16 + r16;
+  const bool col_ok = col < dv;
+  const float* rows = a.vectors + (size_t)row0 * a.width;
+  const float* vcol = rows + 3 * hk + h * dv + (col_ok ? col : 0);
+  float* st = a.state + (size_t)(a.slot_id ? a.slot_id[w] : w) * a.slot_stride +
+              ((size_t)h * dv + (col_ok ? col : 0)) * dk;
+  const bool aligned = dk % 4 == 0 && a.slot_stride % 4 == 0 &&
+                       (reinterpret_cast<uintptr_t>(a.state) & 15) == 0;
+
+  f32x4_t S[NT];
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    S[t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    const int c = t * 16 + 4 * g;
+    if (!a.slot_id || !col_ok) continue;
+    if (aligned) {
+      if (c < dk) S[t] = *reinterpret_cast<const f32x4_t*>(st + c);
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (c + i < dk) S[t][i] = st[c + i];
+    }
+  }
+
+  // this thread's units: channel uc[u], q (first DK units) or k
+  float dec[U][CM_TOKENS], x[U][CM_TOKENS], v[4];
+  float carried[U], since[U];     // L_n of the block before; the product of all decays so far
+  int uc[U];
+  bool is_q[U], unit[U];
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    const int id = tid + u * 256;
+    unit[u] = id < UNITS;
+    is_q[u] = id < DK;
+    uc[u] = is_q[u] ? id : id - DK;
+    carried[u] = since[u] = 1.f;
+  }
+  auto request = [&](int t0) {
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const bool in = unit[u] && uc[u] < dk;
+      const float* ap = rows + (size_t)t0 * a.width + 2 * hk + h * dk + (in ? uc[u] : 0);
+      const float* xp = ap - (is_q[u] ? 2 * hk : hk);
+#pragma unroll
+      for (int i = 0; i < CM_TOKENS; ++i) {
+        const bool ok = in && t0 + i < n_rows;
+        dec[u][i] = ok ? ap[(size_t)i * a.width] : 1.f;
+        x[u][i] = ok ? xp[(size_t)i * a.width] : 0.f;
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      v[j] = col_ok && t0 + 4 * g + j < n_rows ? vcol[(size_t)(t0 + 4 * g + j) * a.width] : 0.f;
+  };
+
+  int n = 0;
+  request(0);
+  for (int t0 = 0; t0 < n_rows; t0 += n) {
+    // ---- L of every token of the block, and where the block ends
+    const int left = n_rows - t0;
+    bool all = true;
+    float L[U][CM_TOKENS];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      float p = 1.f;
+#pragma unroll
+      for (int i = 0; i < CM_TOKENS; ++i) {
+        if (i > 0) p *= dec[u][i];
+        L[u][i] = p;
+      }
+      all = all && p >= CM_FLOOR;
+    }
+    if (tid == 0) shortest = CM_TOKENS;
+    n = left < CM_TOKENS ? left : CM_TOKENS;
+    // (also: every wave is done with the block before)
+    if (!__syncthreads_and(all)) {
+      int fits = CM_TOKENS;
+#pragma unroll
+      for (int u = 0; u < U; ++u)
+#pragma unroll
+        for (int i = CM_TOKENS - 1; i > 0; --i)
+          if (!(L[u][i] >= CM_FLOOR) && i < fits) fits = i;
+      atomicMin(&shortest, fits);
+      __syncthreads();
+      n = shortest < n ? shortest : n;
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      if (!unit[u]) continue;
+      const int c = uc[u];
+      float last = 1.f;
+#pragma unroll
+      for (int i = 0; i < CM_TOKENS; ++i) {
+        const bool in = i < n;
+        if (in) last = L[u][i];
+        const float y = !in ? 0.f : is_q[u] ? x[u][i] * L[u][i] : x[u][i] / L[u][i];
+        if (is_q[u]) {
+          qs[i][c] = y;
+          if (a.scaled_q && blockIdx.z == 0 && in && c < dk)
+            a.scaled_q[(size_t)(row0 + t0 + i) * hk + h * dk + c] =
+                x[u][i] * (since[u] * dec[u][0] * L[u][i]);
+        } else {
+          ks[i][c] = y;
+          kt[c][i] = y;
+        }
+      }
+      if (!is_q[u]) grow[c] = carried[u] * dec[u][0];
+      carried[u] = last;
+      since[u] *= dec[u][0] * last;
+    }
+    float vb[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) vb[j] = 4 * g + j < n ? v[j] : 0.f;
+    __syncthreads();
+    if (t0 + n < n_rows) request(t0 + n);
+
+    // ---- the scores of the block's own tokens, each wave over a quarter of the channels
+    f32x4_t sc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+      if ((t & 3) != wave) continue;
+      const f32x4_t fq = *reinterpret_cast<const f32x4_t*>(&qs[r16][t * 16 + 4 * g]);
+      const f32x4_t fk = *reinterpret_cast<const f32x4_t*>(&ks[r16][t * 16 + 4 * g]);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        sc = __builtin_amdgcn_mfma_f32_16x16x4f32(fq[j], fk[j], sc, 0, 0, 0);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) part[wave][4 * g + i][r16] = sc[i];
+
+    // ---- what the state gives
+    f32x4_t o[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+      const f32x4_t f = *reinterpret_cast<const f32x4_t*>(&grow[t * 16 + 4 * g]);
+      S[t] *= f;
+      const f32x4_t fq = *reinterpret_cast<const f32x4_t*>(&qs[r16][t * 16 + 4 * g]);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        o[t & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(fq[j], S[t][j], o[t & 1], 0, 0, 0);
+    }
+    __syncthreads();
+
+    // ---- what the block's own tokens give
+    f32x4_t p = *reinterpret_cast<const f32x4_t*>(&part[0][r16][4 * g]);
+#pragma unroll
+    for (int q = 1; q < 4; ++q)
+      if (q < NT) p += *reinterpret_cast<const f32x4_t*>(&part[q][r16][4 * g]);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const float pj = 4 * g + j <= r16 ? p[j] : 0.f;
+      o[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(pj, vb[j], o[0], 0, 0, 0);
+    }
+    o[0] += o[1];
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (col_ok && 4 * g + i < n)
+        a.out[(size_t)(row0 + t0 + 4 * g + i) * a.H * dv + h * dv + col] = o[0][i];
+
+    // ---- what they leave in the state
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+      const f32x4_t fk = *reinterpret_cast<const f32x4_t*>(&kt[t * 16 + r16][4 * g]);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        S[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(fk[j], vb[j], S[t], 0, 0, 0);
+    }
+  }
+  __syncthreads();
+#pragma unroll
+  for (int u = 0; u < U; ++u) {
+    if (!unit[u]) continue;
+    if (!is_q[u]) grow[uc[u]] = carried[u];
+    else if (a.total && blockIdx.z == 0 && uc[u] < dk)
+      a.total[(size_t)w * hk + h * dk + uc[u]] = since[u];
+  }
+  __syncthreads();
+  if (!col_ok) return;
+#pragma unroll
+  for (int t = 0; t < NT; ++t) {
+    const int c = t * 16 + 4 * g;
+    const f32x4_t f = *reinterpret_cast<const f32x4_t*>(&grow[c]);
+    S[t] *= f;
+    if (aligned) {
+      if (c < dk) *reinterpret_cast<f32x4_t*>(st + c) = S[t];
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (c + i < dk) st[c + i] = S[t][i];
+    }
+  }
+}
+
+#define CM_MAX_DK 256
+static int launch_channel_blocks(const ChannelArgs& a, int walkers, hipStream_t stream) {
+  dim3 grid(walkers, a.H, (a.dv + 63) / 64), block(256);
+#define ZA_BLOCKS(NT) hipLaunchKernelGGL((channel_blocks_kernel<NT>), grid, block, 0, stream, a)
+  if (a.dk <= 32) ZA_BLOCKS(2);
+  else if (a.dk <= 64) ZA_BLOCKS(4);
+  else if (a.dk <= 128) ZA_BLOCKS(8);
+  else if (a.dk <= CM_MAX_DK) ZA_BLOCKS(16);
+  else return ZA_ERR_UNSUPPORTED;
+#undef ZA_BLOCKS
+  return za_launch_status();
+}
+
+// Every request's portion by one walker from its own state (`vectors` as channel_decay_prepare
+// leaves them): token by token where portions are a few tokens, in blocks otherwise (a function
+// of the step's shape alone, as a recorded step needs it).
 extern "C" int za_channel_recurrence(const float* vectors, int width, float* state,
                                      long long slot_stride, const int* seq_start,
                                      const int* slot_id, float* out, int n_tokens, int n_seqs, int H,
@@ -849,63 +1119,24 @@ extern "C" int za_channel_recurrence(const float* vectors, int width, float* sta
       (lanes & (lanes - 1)) || lanes * RC_ROWS < dk || slot_stride < (long long)H * dk * dv)
     return ZA_ERR_ARG;
   const int hk = H * dk;
+  const bool long_portions = n_tokens > 4 * n_seqs;
+  if (long_portions && dk <= CM_MAX_DK)
+    return launch_channel_blocks(ChannelArgs{vectors, width, state, slot_stride, seq_start, nullptr,
+                                             slot_id, out, nullptr, nullptr, H, dk, dv},
+                                 n_seqs, stream);
   RecurrenceArgs a{vectors, width, 0, hk, 3 * hk, nullptr, 0, 0, 0, nullptr, 0, nullptr, nullptr,
                    nullptr, state, slot_stride, seq_start, slot_id, out, H, H, dk, dv, nullptr,
                    nullptr, 2 * hk};
-  return launch_recurrence<RC_CHANNEL>(a, n_seqs, lanes, n_tokens > 4 * n_seqs, stream);
+  return launch_recurrence<RC_CHANNEL>(a, n_seqs, lanes, long_portions, stream);
 }
 
 // Long portions in chunks, as for the fixed decay: every chunk is walked by itself from an
 // empty state, and what the state before it adds to its read-outs is linear in that state:
-//   1. the walk, one walker a chunk:              o_local[t], the chunk's own final state L_c
-//   2. channel_scan: with A_t the product of the chunk's decays up to and including token t
-//      (at most one, so nothing overflows),       q_t <- q_t * A_t in place;  A_c = A at its end
-//   3. channel_prefix: the state before chunk c,  B_c = diag(A_(c-1)) B_(c-1) + L_(c-1)
-//   4. channel_readout:                           o[t] = o_local[t] + B_c^T (q_t * A_t)
-// 4 is a matrix product and runs on the matrix cores in their 32-bit form
-// (v_mfma_f32_16x16x4_f32: products and sums in full 32-bit).
-
-// A workgroup serves 64 channels of one chunk: 8 waves take an eighth of its tokens each
-// (at most CS_PART), their decays kept in registers between the product and the scaling.
-#define CS_PART 32
-__global__ void __launch_bounds__(512)
-channel_scan_kernel(float* __restrict__ vectors, int width, const int* __restrict__ item_row0,
-                    const int* __restrict__ item_count, float* __restrict__ total, int hk) {
-  __shared__ float part_total[8][64];
-  const int item = blockIdx.x, lane = threadIdx.x & 63, part = threadIdx.x >> 6;
-  const int c = blockIdx.y * 64 + lane;
-  const int row0 = item_row0[item], cnt = item_count[item];
-  const int per = (cnt + 7) / 8, begin = part * per;
-  const int n = cnt - begin < per ? cnt - begin : per;      // (may be negative: no tokens)
-  float* base = vectors + (size_t)(row0 + begin) * width + c;
-  float a[CS_PART];
-  float prod = 1.f;
-#pragma unroll
-  for (int j = 0; j < CS_PART; ++j) a[j] = (c < hk && j < n) ? base[(size_t)j * width + 2 * hk] : 1.f;
-#pragma unroll
-  for (int j = 0; j < CS_PART; ++j) prod *= a[j];
-  part_total[part][lane] = prod;
-  __syncthreads();
-  float before = 1.f, all = 1.f;
-#pragma unroll
-  for (int p = 0; p < 8; ++p) {
-    if (p < part) before *= part_total[p][lane];
-    all *= part_total[p][lane];
-  }
-  if (c >= hk) return;
-  if (part == 0) total[(size_t)item * hk + c] = all;
-#pragma unroll
-  for (int j0 = 0; j0 < CS_PART; j0 += 8) {
-    float q[8];
-#pragma unroll
-    for (int j = 0; j < 8; ++j) q[j] = j0 + j < n ? base[(size_t)(j0 + j) * width] : 0.f;
-#pragma unroll
-    for (int j = 0; j < 8; ++j) {
-      before *= a[j0 + j];
-      if (j0 + j < n) base[(size_t)(j0 + j) * width] = q[j] * before;
-    }
-  }
-}
+//   1. channel_blocks, one walker a chunk:        o_local[t], the chunk's own final state L_c,
+//      with A_t the product of the chunk's decays up to and including token t (at most one, so
+//      nothing overflows) the queries q_t * A_t, and A_c = A at the chunk's end
+//   2. channel_prefix: the state before chunk c,  B_c = diag(A_(c-1)) B_(c-1) + L_(c-1)
+//   3. channel_readout:                           o[t] = o_local[t] + B_c^T (q_t * A_t)
 
 // One thread a state element; the chunks of a request are neighbours in the list.
 __global__ void __launch_bounds__(256)
@@ -961,7 +1192,7 @@ __device__ __forceinline__ f32x4_t four_or_fewer(const float* p, int n, bool ali
 // runs is free as long as both operands agree: slot g of step j is channel 4 g + j of a
 // block of 16, so that a lane's four steps are four neighbouring floats.
 __global__ void __launch_bounds__(256)
-channel_readout_kernel(const float* __restrict__ vectors, int width,
+channel_readout_kernel(const float* __restrict__ scaled_q,
                        const float* __restrict__ chunk_state, const int* __restrict__ item_row0,
                        const int* __restrict__ item_count, float* __restrict__ out, int H, int dk,
                        int dv, int column_blocks) {
@@ -973,9 +1204,9 @@ channel_readout_kernel(const float* __restrict__ vectors, int width,
   const int n0 = (blockIdx.z % column_blocks) * 64;
   if (t0 >= cnt) return;
   const bool row_ok = t0 + r16 < cnt;
-  const float* q = vectors + (size_t)(row0 + (row_ok ? t0 + r16 : 0)) * width + h * dk;
+  const float* q = scaled_q + ((size_t)(row0 + (row_ok ? t0 + r16 : 0)) * H + h) * dk;
   const float* B = chunk_state + ((size_t)item * H + h) * dv * dk;
-  const bool aligned = dk % 4 == 0 && width % 4 == 0;
+  const bool aligned = dk % 4 == 0;
   f32x4_t acc[4];
 #pragma unroll
   for (int j = 0; j < 4; ++j) acc[j] = f32x4_t{0.f, 0.f, 0.f, 0.f};
@@ -1008,44 +1239,36 @@ channel_readout_kernel(const float* __restrict__ vectors, int width,
   }
 }
 
-// `item_*`: the step's work items of at most `chunk` (<= 8 * CS_PART) rows; `iota`: 0 .. n_items
-// - 1; `chunk_state`: n_items * H*dv*dk floats, zero on entry; `total`: n_items * H*dk floats.
-// `vectors`' queries are overwritten.
-extern "C" int za_channel_recurrence_chunked(float* vectors, int width, float* state,
+// `item_*`: the step's work items of at most `chunk` rows; scratch: `chunk_state` n_items *
+// H*dv*dk floats, `scaled_q` n_tokens * H*dk, `total` n_items * H*dk.
+extern "C" int za_channel_recurrence_chunked(const float* vectors, int width, float* state,
                                              long long slot_stride, const int* slot_id,
                                              const int* item_seq, const int* item_row0,
-                                             const int* item_count, const int* iota, int n_items,
-                                             int n_seqs, int chunk, float* chunk_state,
+                                             const int* item_count, int n_items, int n_seqs,
+                                             int chunk, float* chunk_state, float* scaled_q,
                                              float* total, float* out, int n_tokens, int H, int dk,
-                                             int dv, int lanes, hipStream_t stream) {
+                                             int dv, hipStream_t stream) {
   if (n_tokens == 0 || n_items == 0) return 0;
   if (n_tokens < 0 || n_seqs <= 0 || n_items < n_seqs || chunk <= 0 || H <= 0 || dk <= 0 ||
       dv <= 0 || !vectors || !state || !slot_id || !item_seq || !item_row0 || !item_count ||
-      !iota || !chunk_state || !total || !out || width < 3 * H * dk + H * dv || lanes < 1 ||
-      lanes > 64 || (lanes & (lanes - 1)) || lanes * RC_ROWS < dk ||
+      !chunk_state || !scaled_q || !total || !out || width < 3 * H * dk + H * dv ||
       slot_stride < (long long)H * dk * dv)
     return ZA_ERR_ARG;
-  if (chunk > 8 * CS_PART || (long long)H * dk * dv > 0x7fffffffLL) return ZA_ERR_UNSUPPORTED;
-  const int hk = H * dk;
-  const long long elems = (long long)hk * dv;
-  RecurrenceArgs a{vectors, width, 0, hk, 3 * hk, nullptr, 0, 0, 0, nullptr, 0, nullptr, nullptr,
-                   nullptr, chunk_state, elems, item_row0, iota, out, H, H, dk, dv, nullptr,
-                   item_count, 2 * hk};
-  int rc = launch_recurrence<RC_CHANNEL>(a, n_items, lanes, n_tokens > 4 * n_items, stream);
-  if (rc != 0) return rc;
-  hipLaunchKernelGGL(channel_scan_kernel, dim3(n_items, (hk + 63) / 64), dim3(512), 0, stream,
-                     vectors, width, item_row0, item_count, total, hk);
-  rc = za_launch_status();
+  const long long elems = (long long)H * dk * dv;
+  if (dk > CM_MAX_DK || elems > 0x7fffffffLL) return ZA_ERR_UNSUPPORTED;
+  int rc = launch_channel_blocks(ChannelArgs{vectors, width, chunk_state, elems, item_row0,
+                                             item_count, nullptr, out, scaled_q, total, H, dk, dv},
+                                 n_items, stream);
   if (rc != 0) return rc;
   hipLaunchKernelGGL(channel_prefix_kernel, dim3(n_seqs, (unsigned)((elems + 255) / 256)),
                      dim3(256), 0, stream, chunk_state, state, slot_stride, slot_id, item_seq,
-                     n_items, total, (int)elems, hk, dk, dv);
+                     n_items, total, (int)elems, H * dk, dk, dv);
   rc = za_launch_status();
   if (rc != 0) return rc;
   const int column_blocks = (dv + 63) / 64;
   hipLaunchKernelGGL(channel_readout_kernel,
                      dim3(n_items, H, (unsigned)((chunk + 63) / 64 * column_blocks)), dim3(256), 0,
-                     stream, vectors, width, chunk_state, item_row0, item_count, out, H, dk, dv,
+                     stream, scaled_q, chunk_state, item_row0, item_count, out, H, dk, dv,
                      column_blocks);
   return za_launch_status();
 }

@@ -178,9 +178,9 @@ _SIGNATURES = {
                                              c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
                                              c_int, c_void_p],
     ("recurrent", "za_channel_recurrence_chunked"): [c_void_p, c_int, c_void_p, c_longlong, c_void_p,
-                                                     c_void_p, c_void_p, c_void_p, c_void_p, c_int,
-                                                     c_int, c_int, c_void_p, c_void_p, c_void_p,
-                                                     c_int, c_int, c_int, c_int, c_int, c_void_p],
+                                                     c_void_p, c_void_p, c_void_p, c_int, c_int,
+                                                     c_int, c_void_p, c_void_p, c_void_p, c_void_p,
+                                                     c_int, c_int, c_int, c_int, c_void_p],
     ("experts", "za_route_topk"): [c_void_p, c_int, c_void_p, c_int, c_int, c_int, c_int, c_int,
                                    c_float, c_int, c_int, c_void_p, c_void_p, c_void_p],
     ("experts", "za_experts_combine"): [c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int,
@@ -2164,7 +2164,8 @@ def _channel_shapes(vectors, state, state_offset, slot_id, heads, dk, dv):
 def channel_recurrence(vectors: torch.Tensor, state: torch.Tensor, state_offset: int,
                        seq_start: torch.Tensor, slot_id: torch.Tensor, heads: int, dk: int,
                        dv: int) -> torch.Tensor:
-    """``S <- diag(a) S + k v^T;  o = S^T q`` token by token, a decay a head and key channel:
+    """``S <- diag(a) S + k v^T;  o = S^T q``, a decay a head and key channel, token by token
+    or, for portions of more than a few tokens, in blocks of sixteen on the matrix cores (32-bit):
     ``vectors`` as ``channel_decay_prepare`` leaves them, the state of slot ``s`` at ``state[s,
     state_offset:]`` as ``[heads][dv][dk]``.  Returns 32-bit ``[T, heads*dv]``."""
     base, slot_stride, lanes = _channel_shapes(vectors, state, state_offset, slot_id, heads, dk, dv)
@@ -2179,6 +2180,7 @@ def channel_recurrence(vectors: torch.Tensor, state: torch.Tensor, state_offset:
 
 
 CHANNEL_CHUNK = 256            # rows of a work item of the chunked walk with channel decays
+CHANNEL_CHUNK_MAX_DK = 256     # state rows of a head that the block kernel takes
 
 
 def channel_recurrence_chunked(vectors: torch.Tensor, state: torch.Tensor, state_offset: int,
@@ -2188,26 +2190,25 @@ def channel_recurrence_chunked(vectors: torch.Tensor, state: torch.Tensor, state
     (``StepContext.attention_items(CHANNEL_CHUNK)``) cut every request's rows into chunks that
     are walked side by side from empty states; the states before each chunk follow from a short
     pass over the chunks, and what they add to each token's read-out is added afterwards
-    (csrc/recurrent.hip).  ``vectors`` is used up (its queries are overwritten).  Same result as
-    the plain walk up to the order of 32-bit operations."""
+    (csrc/recurrent.hip).  Same result as the plain walk up to the order of 32-bit operations."""
     item_seq, item_row0, item_count, n_items = items
-    base, slot_stride, lanes = _channel_shapes(vectors, state, state_offset, slot_id, heads, dk, dv)
+    base, slot_stride, _ = _channel_shapes(vectors, state, state_offset, slot_id, heads, dk, dv)
     T, S = vectors.shape[0], slot_id.numel()
     for name, t in (("item_seq", item_seq), ("item_row0", item_row0), ("item_count", item_count)):
         _need(t, name, torch.int32)
         if t.numel() < n_items:
             raise KernelError(f"{name} holds {t.numel()} entries, fewer than {n_items} items")
-    if n_items < S:
-        raise KernelError(f"{n_items} items for {S} requests")
+    if n_items < S or dk > CHANNEL_CHUNK_MAX_DK:
+        raise KernelError(f"{n_items} items for {S} requests, dk={dk}")
     dev = vectors.device
     out = torch.empty((T, heads * dv), dtype=torch.float32, device=dev)
-    chunk_state = torch.zeros((n_items, heads * dv * dk), dtype=torch.float32, device=dev)
+    chunk_state = torch.empty((n_items, heads * dv * dk), dtype=torch.float32, device=dev)
+    scaled_q = torch.empty((T, heads * dk), dtype=torch.float32, device=dev)
     total = torch.empty((n_items, heads * dk), dtype=torch.float32, device=dev)
-    iota = torch.arange(n_items, dtype=torch.int32, device=dev)
     rc = _fn("recurrent", "za_channel_recurrence_chunked")(
         _ptr(vectors), vectors.shape[1], base, slot_stride, _ptr(slot_id), _ptr(item_seq),
-        _ptr(item_row0), _ptr(item_count), _ptr(iota), n_items, S, CHANNEL_CHUNK, _ptr(chunk_state),
-        _ptr(total), _ptr(out), T, heads, dk, dv, lanes, _stream())
+        _ptr(item_row0), _ptr(item_count), n_items, S, CHANNEL_CHUNK, _ptr(chunk_state),
+        _ptr(scaled_q), _ptr(total), _ptr(out), T, heads, dk, dv, _stream())
     _check(rc, "channel_recurrence_chunked", f"heads={heads} dk={dk} dv={dv} items={n_items}")
     return out
 

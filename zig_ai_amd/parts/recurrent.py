@@ -373,7 +373,9 @@ class GatedLinearAttention(Mixer):
         self.decay_bias = tensors["decay_up.bias"]
         self.norm_w = tensors["norm.weight"]
         self.w_out = ops.projection_weight(tensors["out_proj.weight"])
-        self.item_granularities = [ops.CHANNEL_CHUNK]
+        # long portions are walked in chunks side by side (the step's work items of that size)
+        self.chunked = d <= ops.CHANNEL_CHUNK_MAX_DK
+        self.item_granularities = [ops.CHANNEL_CHUNK] if self.chunked else []
         ops.check_projection_weight(self.w_in, "gated_linear opening projection")
         ops.check_projection_weight(self.w_out, "gated_linear out_proj")
 
@@ -384,8 +386,8 @@ class GatedLinearAttention(Mixer):
                                             self.decay_bias, self.root, d ** -0.5, H, d, dv)
         if getattr(step, "taps", None) is not None:
             step.taps["vectors"] = vectors.clone()
-        items = step.attention_items(ops.CHANNEL_CHUNK)
-        if items[3] > step.n_seqs:
+        items = step.attention_items(ops.CHANNEL_CHUNK) if self.chunked else None
+        if items is not None and items[3] > step.n_seqs:
             # some request brings more than a chunk (a function of the step's shape alone)
             o = ops.channel_recurrence_chunked(vectors, cache.state, 0, step.slot_id, items, H, d, dv)
         else:
