@@ -276,9 +276,11 @@ def test_random_configurations(seed):
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 def test_chunk_edges(dtype):
     from zig_ai_amd.kernels import ops
-    C = ops.CHANNEL_CHUNK
+    C = ops.CHANNEL_CHUNKS[1]
+    # (the second layer's many heads take the longer chunks, the first the shorter)
     cfg = vu.config([vu.layer("gla", vu.gla(heads=2, dim=20, vdim=24, tau=4.0)),
-                     vu.layer("gla", vu.gla(heads=3, dim=8, vdim=72, tau=1.0, rank=3))], buckets=19)
+                     vu.layer("gla", vu.gla(heads=86, dim=4, vdim=72, tau=1.0, rank=3))], buckets=19)
+    assert [ops.channel_chunk(3, 1, *hv) for hv in ((2, 24), (86, 72))] == list(ops.CHANNEL_CHUNKS)
     model, tensors = build(cfg, seed=6, dtype=dtype)
     lengths = [2 * C + 45, C - 1, C, C + 1, C + 2, 3]
     prompts = [vu.tokens(n, cfg["vocab"], 70 + i) for i, n in enumerate(lengths)]
@@ -665,8 +667,8 @@ def test_trace_replay_and_command_line(tmp_path):
 # ------------------------------------------------------------------ kernels alone
 @pytest.mark.parametrize("H,dk,dv", [(2, 16, 16), (3, 20, 70), (1, 64, 128), (2, 130, 9), (1, 7, 3)])
 def test_channel_recurrence_kernels(H, dk, dv):
-    """The plain walk and the chunked one against float64, from states that are not zero, with
-    decays from one down to exactly zero."""
+    """The blocks and the chunks against float64, from states that are not zero, with decays
+    from one down to exactly zero; then single tokens, which are walked one by one."""
     from zig_ai_amd.engine.batch import _make_items
     from zig_ai_amd.kernels import ops
     dev = torch.device("cuda")
@@ -695,18 +697,24 @@ def test_channel_recurrence_kernels(H, dk, dv):
             want[t] = (S * q[t].double().view(H, dk, 1)).sum(dim=1).reshape(-1)
         after[s, pad:] = S.transpose(1, 2).reshape(-1)
         row += n
-    seq, row0, cnt = _make_items(lens, ops.CHANNEL_CHUNK)
     mk = lambda x: torch.tensor(x, dtype=torch.int32, device=dev)
-    for chunked in (False, True):
+    for chunked in (0,) + ops.CHANNEL_CHUNKS:
         st, vec = state.to(dev), vectors.to(dev)
         if chunked:
+            seq, row0, cnt = _make_items(lens, chunked)
             got = ops.channel_recurrence_chunked(vec, st, pad, slot_id, (mk(seq), mk(row0), mk(cnt), len(seq)),
-                                                 H, dk, dv)
+                                                 chunked, H, dk, dv)
         else:
             got = ops.channel_recurrence(vec, st, pad, start, slot_id, H, dk, dv)
         scale = float(want.abs().max())
         assert float((got.cpu().double() - want).abs().max()) < 1e-5 * scale, chunked
         assert float((st.cpu().double() - after).abs().max()) < 1e-5 * float(after.abs().max()), chunked
+    # the first token of every request, as a step of single tokens
+    first = [int(r) for r in start[:-1]]
+    st = state.to(dev)
+    got = ops.channel_recurrence(vectors[first].contiguous().to(dev), st, pad,
+                                 mk(list(range(len(lens) + 1))), slot_id, H, dk, dv)
+    assert float((got.cpu().double() - want[first]).abs().max()) < 1e-5 * scale
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])

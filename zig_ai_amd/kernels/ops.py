@@ -2179,15 +2179,28 @@ def channel_recurrence(vectors: torch.Tensor, state: torch.Tensor, state_offset:
     return out
 
 
-CHANNEL_CHUNK = 256            # rows of a work item of the chunked walk with channel decays
+# rows of a work item of the chunked walk with channel decays: the longer chunks where they
+# make enough workgroups (two a compute unit), the shorter ones otherwise (16 heads of 128 x 128:
+# one prompt of 2,048 tokens 96 us with chunks of 128 and 118 with 256; of 4,096 tokens 175 and 160)
+CHANNEL_CHUNKS = (128, 256)
+CHANNEL_WORKGROUPS = 512
 CHANNEL_CHUNK_MAX_DK = 256     # state rows of a head that the block kernel takes
 
 
+def channel_chunk(n_long_items: int, n_seqs: int, heads: int, dv: int) -> int:
+    """The chunk for a step that the longer chunks cut into ``n_long_items`` items; 0: no request
+    brings more than one, so nothing is cut."""
+    if n_long_items <= n_seqs:
+        return 0
+    workgroups = n_long_items * heads * ((dv + 63) // 64)
+    return CHANNEL_CHUNKS[1] if workgroups >= CHANNEL_WORKGROUPS else CHANNEL_CHUNKS[0]
+
+
 def channel_recurrence_chunked(vectors: torch.Tensor, state: torch.Tensor, state_offset: int,
-                               slot_id: torch.Tensor, items, heads: int, dk: int,
+                               slot_id: torch.Tensor, items, chunk: int, heads: int, dk: int,
                                dv: int) -> torch.Tensor:
     """``channel_recurrence`` for steps with long portions: ``items``
-    (``StepContext.attention_items(CHANNEL_CHUNK)``) cut every request's rows into chunks that
+    (``StepContext.attention_items(chunk)``) cut every request's rows into chunks that
     are walked side by side from empty states; the states before each chunk follow from a short
     pass over the chunks, and what they add to each token's read-out is added afterwards
     (csrc/recurrent.hip).  Same result as the plain walk up to the order of 32-bit operations."""
@@ -2207,7 +2220,7 @@ def channel_recurrence_chunked(vectors: torch.Tensor, state: torch.Tensor, state
     total = torch.empty((n_items, heads * dk), dtype=torch.float32, device=dev)
     rc = _fn("recurrent", "za_channel_recurrence_chunked")(
         _ptr(vectors), vectors.shape[1], base, slot_stride, _ptr(slot_id), _ptr(item_seq),
-        _ptr(item_row0), _ptr(item_count), n_items, S, CHANNEL_CHUNK, _ptr(chunk_state),
+        _ptr(item_row0), _ptr(item_count), n_items, S, int(chunk), _ptr(chunk_state),
         _ptr(scaled_q), _ptr(total), _ptr(out), T, heads, dk, dv, _stream())
     _check(rc, "channel_recurrence_chunked", f"heads={heads} dk={dk} dv={dv} items={n_items}")
     return out

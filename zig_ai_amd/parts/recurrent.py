@@ -375,7 +375,7 @@ class GatedLinearAttention(Mixer):
         self.w_out = ops.projection_weight(tensors["out_proj.weight"])
         # long portions are walked in chunks side by side (the step's work items of that size)
         self.chunked = d <= ops.CHANNEL_CHUNK_MAX_DK
-        self.item_granularities = [ops.CHANNEL_CHUNK] if self.chunked else []
+        self.item_granularities = list(ops.CHANNEL_CHUNKS) if self.chunked else []
         ops.check_projection_weight(self.w_in, "gated_linear opening projection")
         ops.check_projection_weight(self.w_out, "gated_linear out_proj")
 
@@ -386,10 +386,12 @@ class GatedLinearAttention(Mixer):
                                             self.decay_bias, self.root, d ** -0.5, H, d, dv)
         if getattr(step, "taps", None) is not None:
             step.taps["vectors"] = vectors.clone()
-        items = step.attention_items(ops.CHANNEL_CHUNK) if self.chunked else None
-        if items is not None and items[3] > step.n_seqs:
-            # some request brings more than a chunk (a function of the step's shape alone)
-            o = ops.channel_recurrence_chunked(vectors, cache.state, 0, step.slot_id, items, H, d, dv)
+        # (a function of the step's shape alone; 0 unless some request brings more than a chunk)
+        chunk = ops.channel_chunk(step.attention_items(ops.CHANNEL_CHUNKS[1])[3], step.n_seqs, H,
+                                  dv) if self.chunked else 0
+        if chunk:
+            o = ops.channel_recurrence_chunked(vectors, cache.state, 0, step.slot_id,
+                                               step.attention_items(chunk), chunk, H, d, dv)
         else:
             o = ops.channel_recurrence(vectors, cache.state, 0, step.seq_start, step.slot_id, H, d, dv)
         if getattr(step, "taps", None) is not None:
