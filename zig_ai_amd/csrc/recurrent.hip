@@ -765,7 +765,7 @@ extern "C" int za_retention_chunked(const float* vectors, int width, int q_col, 
 // with the decays a = sigmoid(z)^(1/root), z = up low[t] + bias: `low` the token's `rank` columns
 // of the projection, `up` [H*dk][rank] a second, small product taken here in 32-bit.  The power
 // is taken through the logarithm, log sigmoid(z) = -softplus(-z).
-// grid (tokens / GP_TOKENS, 256 channels).
+// grid (tokens / GP_TOKENS, channels / workgroup size).
 #define GP_TOKENS 8
 #define GP_RANK 256     // columns of `low` staged at a time
 template <typename T, typename TW>
@@ -775,15 +775,23 @@ channel_decay_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_
                              const float* __restrict__ bias, float inv_root, float q_scale,
                              float* __restrict__ out, int out_width, int n_tokens, int hk, int hv) {
   __shared__ float low[GP_TOKENS][GP_RANK];
-  const int t0 = blockIdx.x * GP_TOKENS, c = blockIdx.y * 256 + threadIdx.x;
+  const int bd = blockDim.x;
+  const int t0 = blockIdx.x * GP_TOKENS, c = blockIdx.y * bd + threadIdx.x;
   const int nt = n_tokens - t0 < GP_TOKENS ? n_tokens - t0 : GP_TOKENS;
-  float z[GP_TOKENS];
+  // (what is only converted is requested first; tokens beyond the last repeat it)
+  float z[GP_TOKENS], q[GP_TOKENS], k[GP_TOKENS], v[GP_TOKENS];
 #pragma unroll
-  for (int i = 0; i < GP_TOKENS; ++i) z[i] = 0.f;
+  for (int i = 0; i < GP_TOKENS; ++i) {
+    const T* row = proj + (size_t)(t0 + (i < nt ? i : nt - 1)) * proj_stride;
+    z[i] = 0.f;
+    q[i] = to_f32<T>(row[q_col + (c < hk ? c : 0)]);
+    k[i] = to_f32<T>(row[k_col + (c < hk ? c : 0)]);
+    v[i] = to_f32<T>(row[v_col + (c < hv ? c : 0)]);
+  }
   for (int r0 = 0; r0 < rank; r0 += GP_RANK) {
     const int rn = rank - r0 < GP_RANK ? rank - r0 : GP_RANK;
     __syncthreads();
-    for (int idx = threadIdx.x; idx < GP_TOKENS * rn; idx += 256) {
+    for (int idx = threadIdx.x; idx < GP_TOKENS * rn; idx += bd) {
       const int i = idx / rn, r = idx % rn;
       low[i][r] = i < nt ? to_f32<T>(proj[(size_t)(t0 + i) * proj_stride + low_col + r0 + r]) : 0.f;
     }
@@ -813,14 +821,13 @@ channel_decay_prepare_kernel(const T* __restrict__ proj, int proj_stride, int q_
 #pragma unroll
   for (int i = 0; i < GP_TOKENS; ++i) {
     if (i >= nt) continue;
-    const T* row = proj + (size_t)(t0 + i) * proj_stride;
     float* dst = out + (size_t)(t0 + i) * out_width;
     if (c < hk) {
-      dst[c] = to_f32<T>(row[q_col + c]) * q_scale;
-      dst[hk + c] = to_f32<T>(row[k_col + c]);
+      dst[c] = q[i] * q_scale;
+      dst[hk + c] = k[i];
       dst[2 * hk + c] = expf(-softplus_f(-(z[i] + b)) * inv_root);
     }
-    if (c < hv) dst[3 * hk + c] = to_f32<T>(row[v_col + c]);
+    if (c < hv) dst[3 * hk + c] = v[i];
   }
 }
 
@@ -837,7 +844,8 @@ extern "C" int za_channel_decay_prepare(const void* proj, int dtype, int proj_st
       out_width < 3 * H * dk + H * dv)
     return ZA_ERR_ARG;
   const int hk = H * dk, hv = H * dv, most = hk > hv ? hk : hv;
-  dim3 grid((n_tokens + GP_TOKENS - 1) / GP_TOKENS, (most + 255) / 256), block(256);
+  const int bd = n_tokens <= 64 ? 64 : 256;      // a decode batch: more, smaller workgroups
+  dim3 grid((n_tokens + GP_TOKENS - 1) / GP_TOKENS, (most + bd - 1) / bd), block(bd);
 #define ZA_CDP(T, TW)                                                                          \
   hipLaunchKernelGGL((channel_decay_prepare_kernel<T, TW>), grid, block, 0, stream,            \
                      (const T*)proj, proj_stride, q_col, k_col, v_col, low_col, rank,          \
