@@ -3,7 +3,7 @@ with one block table per request and group, and one slot of fixed-size state
 per request for the mixers that carry state.
 
 Groups.  Mixers declare what they need (``PagedNeed`` or ``StateNeed``).  Paged
-needs that are equal (the same planes per token, window and storage type) form a
+needs that are equal (the same planes per token, window, kept first tokens and storage type) form a
 *group*: its layers
 share one block table per request (page ``p`` names the same place in every
 layer's plane of the group's tensor) and the group has a pool of pages of its
@@ -16,7 +16,7 @@ inside the layer object, which limits it to one live request
 Life of a request: ``admit`` (takes a slot, zeroes its state), then per step
 ``reserve`` (pages for the step's tokens; all or nothing) and ``commit`` (the
 tokens are in the cache; pages wholly behind a group's window go back to the
-pool), finally ``release`` (every page and the slot go back).
+pool, but for those with the first tokens that the group keeps), finally ``release`` (every page and the slot go back).
 
 Device memory: per group one tensor ``[layer, page, elements of a page]``; a page
 holds the group's planes one after the other, plane ``p`` as ``[heads_p, page_size,
@@ -133,6 +133,9 @@ class CacheManager:
                 state_entries.append((cid, need.state))
                 need = need.paged
             if isinstance(need, PagedNeed):
+                if need.window < 0 or need.keep_first < 0:
+                    raise ValueError(f"cache entry {cid!r}: a window of {need.window} and "
+                                     f"{need.keep_first} kept tokens: neither may be negative")
                 if not need.planes or any(h <= 0 or w <= 0 for h, w in need.planes):
                     raise ValueError(f"cache entry {cid!r}: a paged need has planes of positive "
                                      f"sizes, got {need.planes!r}")
@@ -154,8 +157,9 @@ class CacheManager:
             raise ValueError(f"a pool cannot have {num_slots} slots")
         G = len(group_needs)
         windows = (ctypes.c_int * max(G, 1))(*[n.window for n in group_needs])
+        keeps = (ctypes.c_int * max(G, 1))(*[n.keep_first for n in group_needs])
         pages = (ctypes.c_int * max(G, 1))(*group_pages)
-        self._ptr = self._lib.za_cache_new(G, windows, pages, int(page_size), int(num_slots),
+        self._ptr = self._lib.za_cache_new(G, windows, keeps, pages, int(page_size), int(num_slots),
                                            1 if scatter_pages else 0)
         if not self._ptr:
             raise ValueError("the host library refused the cache's sizes")
@@ -388,7 +392,8 @@ class CacheManager:
 
     def stats(self) -> dict:
         return {
-            "groups": [{"window": g.need.window, "layers": len(g.cache_ids),
+            "groups": [{"window": g.need.window, "keep_first": g.need.keep_first,
+                        "layers": len(g.cache_ids),
                         "pages": g.pool.size, "pages_free": g.pool.free_count,
                         "pages_high_water": g.pool.high_water,
                         "pages_taken": g.pool.total_taken} for g in self.groups],

@@ -20,6 +20,7 @@ from .ranesun import RanesunConfig  # noqa: F401
 from .gemodra import GemodraConfig  # noqa: F401
 from .nopozen import NopozenConfig  # noqa: F401
 from .vupelorn import VupelornConfig  # noqa: F401
+from .torisun import TorisunConfig  # noqa: F401
 
 _ARCHITECTURES: Dict[str, Any] = {}
 
@@ -74,3 +75,4 @@ register_architecture("Ranesun", RanesunConfig)
 register_architecture("Gemodra", GemodraConfig)
 register_architecture("Nopozen", NopozenConfig)
 register_architecture("Vupelorn", VupelornConfig)
+register_architecture("Torisun", TorisunConfig)

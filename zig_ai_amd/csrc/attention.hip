@@ -2,7 +2,8 @@
 // prompt portions and single decoded tokens in one launch.
 //
 //   s[t,h,j] = (q[t,h] . k[j,kv(h)]) * scale,  kv(h) = h / (nh / nkv)
-//   keys j <= position(t) only, and j > position(t) - window when window > 0, and
+//   keys j <= position(t) only, and j > position(t) - window (or j < keep: kept first
+//   tokens; the general kernel and attention_planes.hip) when window > 0, and
 //   floor(j / chunk) = floor(position(t) / chunk) when chunk > 0 (the general kernel)
 //   softmax over j in 32-bit, streaming: running maximum m and sum l, the
 //   accumulator rescaled by exp(m_old - m_new) when the maximum moves
@@ -27,33 +28,8 @@
 // matrix-core kernels fetch their value operands with plain 8-byte loads.
 #include <math.h>
 
-#include "common.h"
+#include "attention_common.h"
 #include "rope_math.h"
-
-// What a design may add to the score of a (query, key) pair and to the softmax; every
-// field's zero means "not there", and every kernel of this file takes the struct:
-//   temperature   q at position p counts (1 + qt_coef * ln(floor((p + 1) / qt_every) + 1))
-//                 times (qt_every > 0)
-//   cap           s <- softcap * tanh(s / softcap) after the scale (softcap > 0)
-//   sink          the softmax's denominator also holds exp(sink[head]): a term with no key
-//                 and no value, neither scaled nor capped, counted once however the
-//                 context is cut (the kernel that sees the whole context adds it at its end,
-//                 otherwise the merge of the ranges does)
-//   chunks        positions are counted in chunks of `chunk` from the sequence's start, and
-//                 a query sees the keys of its own chunk only (chunk > 0); in the
-//                 matrix-core kernels the `SHAPED` instantiations know it
-struct ScoreExtras {
-  float softcap;
-  const float* sink;
-  float qt_coef;
-  int qt_every;
-  int chunk;
-};
-
-// first key a query at `position` sees when positions are counted in chunks (0 without)
-__device__ __forceinline__ int chunk_start(const ScoreExtras& ex, int position) {
-  return ex.chunk > 0 && position > 0 ? (position / ex.chunk) * ex.chunk : 0;
-}
 
 __device__ __forceinline__ float query_temperature(const ScoreExtras& ex, int position) {
   if (ex.qt_every <= 0) return 1.0f;
@@ -63,8 +39,6 @@ __device__ __forceinline__ float query_temperature(const ScoreExtras& ex, int po
 __device__ __forceinline__ float capped_score(const ScoreExtras& ex, float s) {
   return ex.softcap > 0.f ? ex.softcap * tanhf(s / ex.softcap) : s;
 }
-
-#define ZA_LOG2E 1.44269504088896341f
 
 // The same for the matrix-core kernels, whose softmax runs on the base-2 scale: the score
 // `dot * row_mul` (row_mul: scale times the row's temperature), capped, times log2(e).
@@ -93,8 +67,6 @@ __device__ __forceinline__ float shaped_score_log2(const ScoreExtras& ex, float 
 #define AT_WAVES 4
 #define AT_RPW 8                     // rows per wave, at most
 #define AT_MAX_ROWS (AT_WAVES * AT_RPW)
-#define AT_MAX_D 256
-#define AT_DPL (AT_MAX_D / 64)       // head-dim elements per lane, at most
 
 template <typename T, int KT>
 __global__ void __launch_bounds__(256)
@@ -141,6 +113,9 @@ paged_attention_kernel(const T* __restrict__ q, T* __restrict__ out, const T* __
   if (range_hi > hi) range_hi = hi;
   int tile_first = (lo / KT) * KT;
   if (tile_first < range_lo) tile_first = range_lo;
+  // kept first keys: their tiles come first, then the walk goes on at the window's
+  const int kept_end = lo > 0 ? (ex.keep + KT - 1) / KT * KT : 0;
+  const int start = kept_end > range_lo ? range_lo : tile_first;
 
   // queries of this item, as floats
   for (int idx = tid; idx < rows * d; idx += 256) {
@@ -159,13 +134,15 @@ paged_attention_kernel(const T* __restrict__ q, T* __restrict__ out, const T* __
   }
 
   const int vec_per_row = d / 8;
-  for (int tile0 = tile_first; tile0 <= range_hi; tile0 += KT) {
+  for (int tile0 = start; tile0 <= range_hi; tile0 += KT) {
+    if (tile0 >= kept_end && tile0 < tile_first) tile0 = tile_first;
+    if (tile0 > range_hi) break;
     __syncthreads();  // previous tile fully consumed (and Qs written, first time)
     for (int idx = tid; idx < KT * vec_per_row; idx += 256) {
       const int j = idx / vec_per_row, c = (idx % vec_per_row) * 8;
       const int kp = tile0 + j;
       float kx[8];
-      bool ok = kp >= lo && kp <= range_hi;
+      bool ok = (kp >= lo || kp < ex.keep) && kp <= range_hi;
       int page = -1;
       if (ok) {
         page = table[kp / page_size];
@@ -186,7 +163,7 @@ paged_attention_kernel(const T* __restrict__ q, T* __restrict__ out, const T* __
       const int j = tid % KT;
       const int kp = tile0 + j;
       const T* vsrc = nullptr;
-      if (kp >= lo && kp <= range_hi) {
+      if ((kp >= lo || kp < ex.keep) && kp <= range_hi) {
         const int page = table[kp / page_size];
         if (page >= 0)
           vsrc = kv + page * page_elems + value_base + (size_t)g * dv * page_size + kp % page_size;
@@ -202,9 +179,10 @@ paged_attention_kernel(const T* __restrict__ q, T* __restrict__ out, const T* __
       if (r < rows) {
         const int pos = positions[row0 + r / G];
         const int kp = tile0 + lane;
-        bool valid = lane < KT && kp <= pos && kp <= range_hi && kp >= lo;
+        bool valid = kp >= lo;
         if (window > 0 && kp <= pos - window) valid = false;
         if (kp < chunk_start(ex, pos)) valid = false;
+        valid = (valid || kp < ex.keep) && lane < KT && kp <= pos && kp <= range_hi;
         float s = -INFINITY;
         if (lane < KT) {
           const float* qr = Qs + r * d;
@@ -284,47 +262,6 @@ paged_attention_kernel(const T* __restrict__ q, T* __restrict__ out, const T* __
   }
 }
 
-// `base2`: the partial maxima are whole numbers on the base-2 scale (what the matrix-core
-// kernels keep), so a partial result's weight 2^(m_z - m) is an exact power of two.
-template <typename T>
-__global__ void __launch_bounds__(64)
-attention_combine_kernel(const float* __restrict__ part_acc, const float* __restrict__ part_ml,
-                         T* __restrict__ out, int d, int nsplit, int base2,
-                         const float* __restrict__ sink, int nh) {
-  // `sink`: one number a head whose exponential joins the denominator once (none if null)
-  const size_t row = blockIdx.x;  // token * nh + head
-  const int lane = threadIdx.x;
-  float mx = -INFINITY;
-  for (int z = 0; z < nsplit; ++z) mx = fmaxf(mx, part_ml[(row * nsplit + z) * 2]);
-  float total = 0.f;
-  float acc[AT_DPL];
-#pragma unroll
-  for (int c = 0; c < AT_DPL; ++c) acc[c] = 0.f;
-  for (int z = 0; z < nsplit; ++z) {
-    const float mz = part_ml[(row * nsplit + z) * 2];
-    const float lz = part_ml[(row * nsplit + z) * 2 + 1];
-    if (!(mz > -INFINITY)) continue;
-    const float w = base2 ? ldexpf(1.0f, (int)(mz - mx)) : expf(mz - mx);
-    total += lz * w;
-    const float* pa = part_acc + (row * nsplit + z) * d;
-#pragma unroll
-    for (int c = 0; c < AT_DPL; ++c) {
-      const int dd = lane + 64 * c;
-      if (dd < d) acc[c] = fmaf(pa[dd], w, acc[c]);
-    }
-  }
-  if (sink && mx > -INFINITY) {
-    const float sk = sink[row % nh];
-    total += base2 ? exp2f(sk * 1.4426950408889634f - mx) : expf(sk - mx);
-  }
-  const float inv = total > 0.f ? 1.0f / total : 0.f;
-#pragma unroll
-  for (int c = 0; c < AT_DPL; ++c) {
-    const int dd = lane + 64 * c;
-    if (dd < d) out[row * d + dd] = from_f32<T>(acc[c] * inv);
-  }
-}
-
 // ------------------------------------------------------------ matrix-core path
 // bfloat16, head_dim 64 or 128, page sizes that are multiples of 4: the same
 // streaming softmax with both products on the matrix cores.
@@ -360,41 +297,6 @@ attention_combine_kernel(const float* __restrict__ part_acc, const float* __rest
 #define AM_ROWS 128
 #define ZA_DECODE_WIDE_BELOW 384   // workgroups: up to here the decode kernel runs eight waves
 
-
-// A query row's scores for a tile are spread over the four lanes l, l ^ 16, l ^ 32,
-// l ^ 48.  The swap instructions exchange 16-lane rows (odd rows of the first operand
-// with even rows of the second) and 32-lane halves between two registers; fed the
-// same value twice they leave in each lane its own value and its partner's, in one
-// vector instruction each and without a trip through LDS.
-__device__ __forceinline__ float quad_max(float x) {
-  const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(x), __float_as_uint(x), false,
-                                                  false);
-  const float y = fmaxf(__uint_as_float(a[0]), __uint_as_float(a[1]));
-  const auto b = __builtin_amdgcn_permlane32_swap(__float_as_uint(y), __float_as_uint(y), false,
-                                                  false);
-  return fmaxf(__uint_as_float(b[0]), __uint_as_float(b[1]));
-}
-__device__ __forceinline__ float quad_sum(float x) {
-  const auto a = __builtin_amdgcn_permlane16_swap(__float_as_uint(x), __float_as_uint(x), false,
-                                                  false);
-  const float y = __uint_as_float(a[0]) + __uint_as_float(a[1]);
-  const auto b = __builtin_amdgcn_permlane32_swap(__float_as_uint(y), __float_as_uint(y), false,
-                                                  false);
-  return __uint_as_float(b[0]) + __uint_as_float(b[1]);
-}
-
-// Key position -> block-table entry and offset in the page.  Page sizes are powers of
-// two nearly always: `shift` is then log2(page_size) and the division (some thirty
-// instructions, several times per tile) becomes a shift; otherwise `shift` is -1.
-__device__ __forceinline__ int page_shift_of(int page_size) {
-  return (page_size & (page_size - 1)) == 0 ? __ffs(page_size) - 1 : -1;
-}
-__device__ __forceinline__ int page_entry(int kp, int page_size, int shift) {
-  return shift >= 0 ? kp >> shift : kp / page_size;
-}
-__device__ __forceinline__ int page_offset(int kp, int page_size, int shift) {
-  return shift >= 0 ? kp & (page_size - 1) : kp % page_size;
-}
 
 template <int D, int NW, int NS, int KT, bool SHAPED>
 __global__ void __launch_bounds__(NW * 64)
@@ -1357,15 +1259,17 @@ static int paged_attention_any(const void* q, void* out, const void* kv, const i
 }
 
 // Everything the general kernel knows, at once: values of width `dv`, an output gate a head
-// or (`gate_elem`) an element, what `ScoreExtras` describes, a window and chunks.
+// or (`gate_elem`) an element, what `ScoreExtras` describes, a window, kept first keys and
+// chunks.
 extern "C" int za_paged_attention_general(
     const void* q, void* out, const void* kv, const int* block_table, int bt_stride,
     const int* positions, const int* wi_seq, const int* wi_row0, const int* wi_count, int n_items,
     int n_tokens, float* part_acc, float* part_ml, int dtype, int nh, int nkv, int d, int dv,
     int page_size, float scale, int window, int keys_per_split, int nsplit, const void* gate,
     int gate_stride, int gate_col, int gate_elem, float out_scale, float softcap,
-    const float* sink, float qt_coef, int qt_every, int chunk, hipStream_t stream) {
-  if (dv <= 0 || dv % 8 != 0 || dv > AT_MAX_D || softcap < 0.f || qt_every < 0 || chunk < 0)
+    const float* sink, float qt_coef, int qt_every, int chunk, int keep, hipStream_t stream) {
+  if (dv <= 0 || dv % 8 != 0 || dv > AT_MAX_D || softcap < 0.f || qt_every < 0 || chunk < 0 ||
+      keep < 0)
     return ZA_ERR_UNSUPPORTED;
   if (gate && (gate_col < 0 || gate_col + (gate_elem ? nh * dv : nh) > gate_stride))
     return ZA_ERR_ARG;
@@ -1373,7 +1277,7 @@ extern "C" int za_paged_attention_general(
                              wi_count, n_items, n_tokens, part_acc, part_ml, dtype, nh, nkv, d,
                              page_size, scale, window, keys_per_split, nsplit, dv, gate,
                              gate_stride, gate_col, out_scale,
-                             ScoreExtras{softcap, sink, qt_coef, qt_every, chunk}, stream,
+                             ScoreExtras{softcap, sink, qt_coef, qt_every, chunk, keep}, stream,
                              gate_elem);
 }
 

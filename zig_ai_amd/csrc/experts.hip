@@ -504,7 +504,7 @@ route_topk_kernel(const float* __restrict__ z, int ld, const float* __restrict__
     }
     __syncthreads();
   }
-  const float f = renorm ? scale / total : scale;
+  const float f = renorm ? scale / (total + 1e-20f) : scale;   // (all scores may underflow)
   for (int j = lane; j < top; j += 64) weight[(size_t)t * top + j] *= f;
 }
 

@@ -839,12 +839,34 @@ gemm_bf16_rows16_gated_conv_kernel(NormedRowsArg normed, const bf16_t* __restric
 //   C[m, n] = silu(gate[m, n]) * up[m, n],   silu(g) = g / (1 + exp(-g)),
 // from the 32-bit accumulators (/root/reference/src/transformer/ffn.zig:24-30), so
 // the [M, 2I] intermediate never goes to memory.  K is not split over workgroups.
+//
+// The unit's form: `act` 0 = silu, 1 = the tanh form of gelu on the gate, times up;
+// 2 = bounded:  g * sigmoid(slope * g) * (u + offset),  g = min(gate, bound),
+// u = clamp(up, -bound, bound)  (bound <= 0: none).
+struct GateForm {
+  int act;
+  float bound, slope, offset;
+};
+
+__device__ __forceinline__ float gate_unit(const GateForm& f, float g, float u) {
+  if (f.act == 2) {
+    if (f.bound > 0.f) {
+      g = fminf(g, f.bound);
+      u = fminf(fmaxf(u, -f.bound), f.bound);
+    }
+    return g * (1.0f / (1.0f + expf(-f.slope * g))) * (u + f.offset);
+  }
+  const float a = f.act == 1
+                      ? 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)))
+                      : g * (1.0f / (1.0f + expf(-g)));
+  return a * u;
+}
+
 template <int NW, int KSTEPS, bool NORM, bool STAGED>
 __global__ void __launch_bounds__(NW * 64, 2)
 gemm_bf16_rows16_swiglu_kernel(const bf16_t* __restrict__ A, NormedRowsArg normed,
                                const bf16_t* __restrict__ W, bf16_t* __restrict__ C, int M, int I,
-                               int K, int groups_per_block, int act) {
-  // `act`: the gate's activation, 0 = silu, 1 = the tanh form of gelu
+                               int K, int groups_per_block, GateForm form) {
   __shared__ float red[2][2][NW][64][4];
   __shared__ float ssw[NW][16];
   const int tid = threadIdx.x;
@@ -977,10 +999,7 @@ gemm_bf16_rows16_swiglu_kernel(const bf16_t* __restrict__ A, NormedRowsArg norme
             gv *= scale;
             uv *= scale;
           }
-          const float gated =
-              act == 1 ? 0.5f * gv * (1.0f + tanhf(0.7978845608028654f * (gv + 0.044715f * gv * gv * gv)))
-                       : gv * (1.0f / (1.0f + expf(-gv)));
-          C[(size_t)m * I + n] = (bf16_t)(gated * uv);
+          C[(size_t)m * I + n] = (bf16_t)gate_unit(form, gv, uv);
         }
       }
     }
@@ -1235,9 +1254,10 @@ extern "C" int za_gemm_bf16_rows16_merged(const float* part_acc, const float* pa
 // za_gemm_bf16_rows16_stream.
 static int rows16_gated_any(const void* A, const float* x, const int* rows,
                             const float* norm_weight, float eps, const void* W, void* C, int M,
-                            int I, int K, int act, hipStream_t stream) {
+                            int I, int K, GateForm form, hipStream_t stream) {
   if (M == 0 || I == 0) return 0;
-  if (M < 0 || I < 0 || K <= 0 || !W || !C || (!A && !x) || act < 0 || act > 1) return ZA_ERR_ARG;
+  if (M < 0 || I < 0 || K <= 0 || !W || !C || (!A && !x) || form.act < 0 || form.act > 2)
+    return ZA_ERR_ARG;
   if (M > 16 || K % 8 != 0 || K > 8192) return ZA_ERR_UNSUPPORTED;
   const bool norm = !A;
   if (norm && (!norm_weight || !rows16_takes_norm(K, 1))) return ZA_ERR_UNSUPPORTED;
@@ -1254,7 +1274,7 @@ static int rows16_gated_any(const void* A, const float* x, const int* rows,
     auto kernel = gemm_bf16_rows16_swiglu_kernel<NW, KS, NORM, STAGED>;                       \
     if (const int rc = rows16_allow_lds((const void*)kernel, lds)) return rc;                         \
     hipLaunchKernelGGL(kernel, grid, dim3(NW * 64), lds, stream, (const bf16_t*)A, normed,    \
-                       (const bf16_t*)W, (bf16_t*)C, M, I, K, per_block, act);                \
+                       (const bf16_t*)W, (bf16_t*)C, M, I, K, per_block, form);               \
   }
 #define ZA_SG_CASE(NW, KS)                                                                    \
   {                                                                                           \
@@ -1278,15 +1298,17 @@ static int rows16_gated_any(const void* A, const float* x, const int* rows,
 extern "C" int za_gemm_bf16_rows16_swiglu(const void* A, const float* x, const int* rows,
                                           const float* norm_weight, float eps, const void* W,
                                           void* C, int M, int I, int K, hipStream_t stream) {
-  return rows16_gated_any(A, x, rows, norm_weight, eps, W, C, M, I, K, 0, stream);
+  return rows16_gated_any(A, x, rows, norm_weight, eps, W, C, M, I, K, GateForm{0, 0.f, 0.f, 0.f},
+                          stream);
 }
 
-// The same with the gate's activation named: 0 = silu, 1 = the tanh form of gelu.
+// The same with the unit's form named (`GateForm`).
 extern "C" int za_gemm_bf16_rows16_gated(const void* A, const float* x, const int* rows,
                                          const float* norm_weight, float eps, const void* W,
-                                         void* C, int M, int I, int K, int act,
-                                         hipStream_t stream) {
-  return rows16_gated_any(A, x, rows, norm_weight, eps, W, C, M, I, K, act, stream);
+                                         void* C, int M, int I, int K, int act, float bound,
+                                         float slope, float offset, hipStream_t stream) {
+  return rows16_gated_any(A, x, rows, norm_weight, eps, W, C, M, I, K,
+                          GateForm{act, bound, slope, offset}, stream);
 }
 
 // The ShortConv mixer from the 32-bit stream to the convolution's output in one kernel

@@ -134,6 +134,7 @@ struct Pool {
 // ------------------------------------------------------------------ cache
 struct Group {
   int window = 0;
+  int keep_first = 0;          // with a window: the first tokens that stay readable all the same
   Pool pool;
   std::vector<char> ever_used;
 };
@@ -215,12 +216,13 @@ struct Cache {
     for (size_t g = 0; g < groups.size(); ++g) {
       const int w = groups[g].window;
       if (w <= 0) continue;
-      // the next query sits at position >= num_tokens and reads keys > position - w
+      // the next query sits at position >= num_tokens and reads keys > position - w, and the
+      // first `keep_first` keys, whose pages (the last of them in part) stay
       const int first_needed = rc->num_tokens - w + 1;
       if (first_needed <= 0) continue;
       auto& table = rc->tables[g];
       const int upto = std::min(first_needed / page_size, (int)table.size());
-      for (int p = 0; p < upto; ++p)
+      for (int p = (groups[g].keep_first + page_size - 1) / page_size; p < upto; ++p)
         if (table[p] != FREED) {
           if (int e = groups[g].pool.give(table[p], req)) return e;
           table[p] = FREED;
@@ -483,16 +485,19 @@ ZA_EXPORT int za_pool_owner(void* p, int item, int64_t* owner) {
 }
 
 // ---- cache
+// `keep_first` (may be null: none): per group, the first tokens that stay behind its window.
 // `scatter_pages`: see Pool::init (slots are never scattered).
-ZA_EXPORT void* za_cache_new(int n_groups, const int* windows, const int* num_pages, int page_size,
-                             int num_slots, int scatter_pages) {
+ZA_EXPORT void* za_cache_new(int n_groups, const int* windows, const int* keep_first,
+                             const int* num_pages, int page_size, int num_slots,
+                             int scatter_pages) {
   if (n_groups < 0 || page_size <= 0 || num_slots < 0) return nullptr;
   Cache* c = new Cache();
   c->page_size = page_size;
   c->groups.resize(n_groups);
   for (int g = 0; g < n_groups; ++g) {
-    if (num_pages[g] < 0) { delete c; return nullptr; }
+    if (num_pages[g] < 0 || (keep_first && keep_first[g] < 0)) { delete c; return nullptr; }
     c->groups[g].window = windows[g];
+    c->groups[g].keep_first = keep_first ? keep_first[g] : 0;
     c->groups[g].pool.init(num_pages[g], true, scatter_pages != 0);
     c->groups[g].ever_used.assign(num_pages[g], 0);
   }

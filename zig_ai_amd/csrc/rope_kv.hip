@@ -27,10 +27,10 @@ qk_norm_rope_kv_write_kernel(const T* __restrict__ qkv, const int* __restrict__ 
                              const float* __restrict__ k_norm_w, const float* __restrict__ inv_freq,
                              T* __restrict__ q_out, T* __restrict__ kv_cache, int nh, int nkv, int d,
                              int rot, int adjacent, float eps, int page_size, int write_kv, int dv,
-                             int row_stride) {
+                             int row_stride, float magnitude) {
   // `dv`: width of a value head (queries and keys have `d`); a row of `qkv` holds
   // nh*d + nkv*d + nkv*dv elements (and may be longer: `row_stride`), a page the keys of
-  // all heads and then the values of all heads.
+  // all heads and then the values of all heads.  `magnitude`: factor on cosine and sine.
   __shared__ float vec[4][RK_MAX_D];
   const int t = blockIdx.x;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
@@ -70,6 +70,8 @@ qk_norm_rope_kv_write_kernel(const T* __restrict__ qkv, const int* __restrict__ 
       const float angle = pos * inv_freq[p];
       float sn, cs;
       sincosf(angle, &sn, &cs);
+      cs *= magnitude;
+      sn *= magnitude;
       const float a = s[i0], b = s[i1];
       s[i0] = a * cs - b * sn;
       s[i1] = a * sn + b * cs;
@@ -298,30 +300,31 @@ extern "C" int za_qk_norm_rope_kv_write(const void* qkv, const int* positions, c
     hipLaunchKernelGGL((qk_norm_rope_kv_write_kernel<float>), grid, block, 0, stream,
                        (const float*)qkv, positions, slots, q_norm_w, k_norm_w, inv_freq,
                        (float*)q_out, (float*)kv_cache, nh, nkv, d, rot, adjacent, eps, page_size,
-                       write_kv, d, (nh + 2 * nkv) * d);
+                       write_kv, d, (nh + 2 * nkv) * d, 1.0f);
   } else if (dtype == 1) {
     hipLaunchKernelGGL((qk_norm_rope_kv_write_kernel<bf16_t>), grid, block, 0, stream,
                        (const bf16_t*)qkv, positions, slots, q_norm_w, k_norm_w, inv_freq,
                        (bf16_t*)q_out, (bf16_t*)kv_cache, nh, nkv, d, rot, adjacent, eps,
-                       page_size, write_kv, d, (nh + 2 * nkv) * d);
+                       page_size, write_kv, d, (nh + 2 * nkv) * d, 1.0f);
   } else {
     return ZA_ERR_UNSUPPORTED;
   }
   return za_launch_status();
 }
 
-// The same for values of another width than the keys' (`dv`) and rows of `qkv` that hold
-// more than q|k|v (`row_stride` elements a row: a gate's columns behind them, say).
+// The same for values of another width than the keys' (`dv`), rows of `qkv` that hold
+// more than q|k|v (`row_stride` elements a row: a gate's columns behind them, say), and a factor
+// `magnitude` on cosine and sine.  nkv == 0: the rows hold queries only, nothing is stored.
 extern "C" int za_qk_norm_rope_kv_write_wide(const void* qkv, const int* positions,
                                              const int* slots, const float* q_norm_w,
                                              const float* k_norm_w, const float* inv_freq,
                                              void* q_out, void* kv_cache, int dtype, int n_tokens,
                                              int nh, int nkv, int d, int dv, int row_stride,
                                              int rot, int adjacent, float eps, int page_size,
-                                             int write_kv, hipStream_t stream) {
+                                             int write_kv, float magnitude, hipStream_t stream) {
   if (n_tokens == 0) return 0;
-  if (n_tokens < 0 || nh <= 0 || nkv <= 0 || d <= 0 || dv <= 0 || !qkv || !positions || !q_out ||
-      row_stride < (nh + nkv) * d + nkv * dv)
+  if (n_tokens < 0 || nh <= 0 || nkv < 0 || d <= 0 || dv <= 0 || !qkv || !positions || !q_out ||
+      row_stride < (nh + nkv) * d + nkv * dv || (nkv == 0 && write_kv))
     return ZA_ERR_ARG;
   if (d > RK_MAX_D || dv > RK_MAX_D || rot < 0 || rot > d || (rot % 2) != 0)
     return ZA_ERR_UNSUPPORTED;
@@ -332,14 +335,201 @@ extern "C" int za_qk_norm_rope_kv_write_wide(const void* qkv, const int* positio
     hipLaunchKernelGGL((qk_norm_rope_kv_write_kernel<float>), grid, block, 0, stream,
                        (const float*)qkv, positions, slots, q_norm_w, k_norm_w, inv_freq,
                        (float*)q_out, (float*)kv_cache, nh, nkv, d, rot, adjacent, eps, page_size,
-                       write_kv, dv, row_stride);
+                       write_kv, dv, row_stride, magnitude);
   } else if (dtype == 1) {
     hipLaunchKernelGGL((qk_norm_rope_kv_write_kernel<bf16_t>), grid, block, 0, stream,
                        (const bf16_t*)qkv, positions, slots, q_norm_w, k_norm_w, inv_freq,
                        (bf16_t*)q_out, (bf16_t*)kv_cache, nh, nkv, d, rot, adjacent, eps,
-                       page_size, write_kv, dv, row_stride);
+                       page_size, write_kv, dv, row_stride, magnitude);
   } else {
     return ZA_ERR_UNSUPPORTED;
   }
   return za_launch_status();
+}
+
+// Queries and keys normed over their WHOLE projection instead of head by head:
+//   q row [nh * d]:  x <- x / sqrt(sum(x^2) / q_count + eps) * q_norm_w[nh * d]
+//   k row [nkv * d]: likewise with k_count and k_norm_w[nkv * d]
+// (q_count, k_count: how many elements the mean is taken over, fewer than the row has where
+// heads are filled up with zeros), then the rotation of every head and the stores of the
+// kernels above, `dv`, `row_stride` and `magnitude` as there.  nkv == 0: the rows hold queries
+// only, nothing is stored (a layer that reads another layer's keys and values).
+//
+// A workgroup a token.  The row's heads are staged in LDS as floats, pieces of eight elements a
+// thread; the two sums of squares meet once, every thread then norms its own pieces, and the
+// rotation reads a piece and its partners from LDS.  In steps of many tokens the values are
+// stored by workgroups of their own, first in the grid: a wave takes eight consecutive tokens
+// and, where these lie side by side in one page, stores a head-dim element's eight values with
+// one access.
+template <typename T>
+__global__ void __launch_bounds__(256)
+qk_row_norm_rope_kv_write_kernel(const T* __restrict__ qkv, const int* __restrict__ positions,
+                                 const int* __restrict__ slots, const float* __restrict__ q_norm_w,
+                                 const float* __restrict__ k_norm_w,
+                                 const float* __restrict__ inv_freq, T* __restrict__ q_out,
+                                 T* __restrict__ kv_cache, int nh, int nkv, int d, int dv,
+                                 int row_stride, int rot, int adjacent, float eps, float q_count,
+                                 float k_count, float magnitude, int page_size, int write_kv,
+                                 int n_tokens, int value_blocks) {
+  extern __shared__ __attribute__((aligned(16))) float rows_lds[];   // [(nh + nkv) * d][rot]
+  __shared__ float sums[2][4];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const size_t page_elems = (size_t)nkv * page_size * (d + dv);
+  const size_t value_base = (size_t)nkv * page_size * d;
+  if ((int)blockIdx.x < value_blocks) {
+    const int t0 = ((int)blockIdx.x * 4 + wave) * 8;   // a wave's 8 tokens
+    if (t0 >= n_tokens) return;
+    int slot[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) slot[j] = t0 + j < n_tokens ? slots[t0 + j] : -1;
+    bool side_by_side = page_size % 8 == 0 && slot[0] >= 0 && slot[0] % 8 == 0;
+#pragma unroll
+    for (int j = 1; j < 8; ++j) side_by_side = side_by_side && slot[j] == slot[0] + j;
+    const int pieces = nkv * dv / 8;
+    for (int piece = lane; piece < pieces; piece += 64) {
+      float x[8][8];
+#pragma unroll
+      for (int j = 0; j < 8; ++j)
+        if (t0 + j < n_tokens)
+          load8<T>(qkv + (size_t)(t0 + j) * row_stride + (size_t)(nh + nkv) * d + piece * 8, x[j]);
+      if (side_by_side) {
+        T* dst = kv_cache + (size_t)(slot[0] / page_size) * page_elems + value_base +
+                 (size_t)piece * 8 * page_size + slot[0] % page_size;
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          float run[8];
+#pragma unroll
+          for (int j = 0; j < 8; ++j) run[j] = x[j][i];
+          store8<T>(dst + (size_t)i * page_size, run);
+        }
+      } else {
+#pragma unroll
+        for (int j = 0; j < 8; ++j)
+          if (slot[j] >= 0) {
+            T* dst = kv_cache + (size_t)(slot[j] / page_size) * page_elems + value_base +
+                     (size_t)piece * 8 * page_size + slot[j] % page_size;
+#pragma unroll
+            for (int i = 0; i < 8; ++i) dst[(size_t)i * page_size] = from_f32<T>(x[j][i]);
+          }
+      }
+    }
+    return;
+  }
+  const int t = (int)blockIdx.x - value_blocks;
+  const T* row = qkv + (size_t)t * row_stride;
+  const int half = rot / 2;
+  const int q_pieces = nh * d / 8;
+  const int pieces = q_pieces + (write_kv ? nkv * d / 8 : 0);
+  float* cs_tab = rows_lds + (size_t)(nh + nkv) * d;
+  float* sn_tab = cs_tab + half;
+
+  float qs = 0.f, ks = 0.f;
+  for (int piece = tid; piece < pieces; piece += 256) {
+    float x[8];
+    load8<T>(row + piece * 8, x);
+    const float ss = rope_sum_squares8(x);
+    if (piece < q_pieces) qs += ss; else ks += ss;
+    store8<float>(rows_lds + piece * 8, x);
+  }
+  for (int p = tid; p < half; p += 256) {
+    float cs, sn;
+    rope_angle(positions[t], inv_freq[p], &cs, &sn);
+    cs_tab[p] = cs * magnitude;
+    sn_tab[p] = sn * magnitude;
+  }
+  qs = wave_sum(qs);
+  ks = wave_sum(ks);
+  if (lane == 0) {
+    sums[0][wave] = qs;
+    sums[1][wave] = ks;
+  }
+  __syncthreads();
+  const float q_scale =
+      1.0f / sqrtf((sums[0][0] + sums[0][1] + sums[0][2] + sums[0][3]) / q_count + eps);
+  const float k_scale =
+      1.0f / sqrtf((sums[1][0] + sums[1][1] + sums[1][2] + sums[1][3]) / k_count + eps);
+  for (int piece = tid; piece < pieces; piece += 256) {
+    const bool is_q = piece < q_pieces;
+    float x[8], w[8];
+    load8<float>(rows_lds + piece * 8, x);
+    load8<float>(is_q ? q_norm_w + piece * 8 : k_norm_w + (piece - q_pieces) * 8, w);
+    rope_scale8(x, is_q ? q_scale : k_scale, w);
+    store8<float>(rows_lds + piece * 8, x);
+  }
+  __syncthreads();
+  const int slot = write_kv ? slots[t] : -1;
+  T* pg = slot >= 0 ? kv_cache + (size_t)(slot / page_size) * page_elems : nullptr;
+  const int off = slot >= 0 ? slot % page_size : 0;
+  for (int piece = tid; piece < pieces; piece += 256) {
+    const int head = piece * 8 / d, e0 = piece * 8 % d;
+    const float* h = rows_lds + (size_t)head * d;
+    float x[8];
+    load8<float>(h + e0, x);
+    if (e0 < rot) {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const int e = e0 + i;
+        if (e >= rot) continue;
+        if (adjacent) {
+          const float other = h[e ^ 1], cs = cs_tab[e >> 1], sn = sn_tab[e >> 1];
+          x[i] = (e & 1) ? rope_rotate_high(x[i], other, cs, sn) : rope_rotate_low(x[i], other, cs, sn);
+        } else if (e < half) {
+          x[i] = rope_rotate_low(x[i], h[e + half], cs_tab[e], sn_tab[e]);
+        } else {
+          x[i] = rope_rotate_high(x[i], h[e - half], cs_tab[e - half], sn_tab[e - half]);
+        }
+      }
+    }
+    if (piece < q_pieces)
+      store8<T>(q_out + (size_t)t * nh * d + piece * 8, x);
+    else if (pg)
+      store8<T>(pg + ((size_t)(head - nh) * page_size + off) * d + e0, x);
+  }
+  if (pg && value_blocks == 0) {
+    const T* v = row + (size_t)(nh + nkv) * d;
+    for (int i = tid; i < nkv * dv; i += 256) pg[value_base + (size_t)i * page_size + off] = v[i];
+  }
+}
+
+#define RK_ROW_MAX_LDS (128 * 1024)
+
+extern "C" int za_qk_row_norm_rope_kv_write(const void* qkv, const int* positions, const int* slots,
+                                            const float* q_norm_w, const float* k_norm_w,
+                                            const float* inv_freq, void* q_out, void* kv_cache,
+                                            int dtype, int n_tokens, int nh, int nkv, int d, int dv,
+                                            int row_stride, int rot, int adjacent, float eps,
+                                            float q_count, float k_count, float magnitude,
+                                            int page_size, int write_kv, hipStream_t stream) {
+  if (n_tokens == 0) return 0;
+  if (n_tokens < 0 || nh <= 0 || nkv < 0 || d <= 0 || dv <= 0 || !qkv || !positions || !q_out ||
+      !q_norm_w || row_stride < (nh + nkv) * d + nkv * dv || !(q_count > 0.f))
+    return ZA_ERR_ARG;
+  if (d % 8 != 0 || dv % 8 != 0 || row_stride % 8 != 0 || rot < 0 || rot > d || rot % 2 != 0)
+    return ZA_ERR_UNSUPPORTED;
+  if (rot > 0 && !inv_freq) return ZA_ERR_ARG;
+  if (write_kv && (nkv == 0 || !kv_cache || !slots || !k_norm_w || page_size <= 0 || !(k_count > 0.f)))
+    return ZA_ERR_ARG;
+  const size_t shmem = ((size_t)(nh + nkv) * d + rot) * sizeof(float);
+  if (shmem > RK_ROW_MAX_LDS) return ZA_ERR_UNSUPPORTED;
+  const int value_blocks = (write_kv && n_tokens >= RK_VALUE_BLOCKS_FROM) ? (n_tokens + 31) / 32 : 0;
+#define ZA_RK_ROW(T)                                                                             \
+  {                                                                                              \
+    auto kernel = qk_row_norm_rope_kv_write_kernel<T>;                                           \
+    static size_t allowed = 48 * 1024;                                                           \
+    if (shmem > allowed) {                                                                       \
+      const hipError_t e = hipFuncSetAttribute(                                                  \
+          (const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)shmem);          \
+      if (e != hipSuccess) return (int)e;                                                        \
+      allowed = shmem;                                                                           \
+    }                                                                                            \
+    hipLaunchKernelGGL(kernel, dim3(n_tokens + value_blocks), dim3(256), shmem, stream,          \
+                       (const T*)qkv, positions, slots, q_norm_w, k_norm_w, inv_freq, (T*)q_out, \
+                       (T*)kv_cache, nh, nkv, d, dv, row_stride, rot, adjacent, eps, q_count,    \
+                       k_count, magnitude, page_size, write_kv, n_tokens, value_blocks);         \
+    return za_launch_status();                                                                   \
+  }
+  if (dtype == 0) ZA_RK_ROW(float)
+  if (dtype == 1) ZA_RK_ROW(bf16_t)
+#undef ZA_RK_ROW
+  return ZA_ERR_UNSUPPORTED;
 }

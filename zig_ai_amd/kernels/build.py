@@ -27,7 +27,7 @@ from typing import Dict, Iterable, List, Optional
 PACKAGE_DIR = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 CSRC_DIR = os.path.join(PACKAGE_DIR, "csrc")
 ARCH = "gfx950"
-SOURCES = ("norm", "gemm", "gemm_rows64", "rope_kv", "attention", "shortconv", "recurrent",
+SOURCES = ("norm", "gemm", "gemm_rows64", "rope_kv", "attention", "attention_planes", "shortconv", "recurrent",
            "activation", "experts", "latent", "sampling", "blaslt", "calibrate")
 HOST_SOURCES = ("host", "plain")    # plain C++, no device code: usable without a GPU or ROCm
 ALL_SOURCES = SOURCES + HOST_SOURCES
@@ -40,8 +40,8 @@ HIPCC_FLAGS = [
 
 EXTRA_FLAGS = {"blaslt": ["-lhipblaslt"]}   # host code around the GEMM library, no kernels
 # headers a source includes beside common.h
-EXTRA_HEADERS = {"sampling": ["no_alloc.h"], "rope_kv": ["rope_math.h"], "attention": ["rope_math.h"],
-                 "recurrent": ["rope_math.h"]}
+EXTRA_HEADERS = {"sampling": ["no_alloc.h"], "rope_kv": ["rope_math.h"], "attention": ["attention_common.h", "rope_math.h"],
+                 "attention_planes": ["attention_common.h"], "recurrent": ["rope_math.h"]}
 
 _loaded: Dict[str, ctypes.CDLL] = {}
 _lock = threading.Lock()

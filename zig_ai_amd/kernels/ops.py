@@ -73,7 +73,7 @@ _SIGNATURES = {
                                              c_void_p, c_void_p, c_int, c_int, c_int, c_void_p],
     ("gemm", "za_gemm_bf16_rows16_gated"): [c_void_p, c_void_p, c_void_p, c_void_p, c_float,
                                             c_void_p, c_void_p, c_int, c_int, c_int, c_int,
-                                            c_void_p],
+                                            c_float, c_float, c_float, c_void_p],
     ("gemm", "za_gemm_bf16_rows16_gated_conv"): [c_void_p, c_void_p, c_void_p, c_float, c_void_p,
                                                  c_void_p, c_void_p, c_void_p, c_longlong,
                                                  c_void_p, c_void_p, c_int, c_int, c_int, c_int,
@@ -92,7 +92,15 @@ _SIGNATURES = {
     ("rope_kv", "za_qk_norm_rope_kv_write_wide"): [c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
                                                    c_void_p, c_void_p, c_void_p, c_int, c_int,
                                                    c_int, c_int, c_int, c_int, c_int, c_int, c_int,
-                                                   c_float, c_int, c_int, c_void_p],
+                                                   c_float, c_int, c_int, c_float, c_void_p],
+    ("rope_kv", "za_qk_row_norm_rope_kv_write"): [
+        c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int,
+        c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_float, c_float,
+        c_int, c_int, c_void_p],
+    ("attention_planes", "za_planes_attention"): [
+        c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
+        c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_float, c_int, c_int,
+        c_int, c_int, c_int, c_void_p, c_void_p],
     ("attention", "za_paged_attention_gated"): [c_void_p, c_void_p, c_void_p, c_void_p, c_int,
                                                 c_void_p, c_void_p, c_void_p, c_void_p, c_int,
                                                 c_int, c_void_p, c_void_p, c_int, c_int, c_int,
@@ -136,7 +144,7 @@ _SIGNATURES = {
         c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_void_p,
         c_int, c_int, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_int,
         c_int, c_int, c_void_p, c_int, c_int, c_int, c_float, c_float, c_void_p, c_float,
-        c_int, c_int, c_void_p],
+        c_int, c_int, c_int, c_void_p],
     ("recurrent", "za_retention_prepare"): [c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p,
                                             c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
                                             c_float, c_void_p],
@@ -912,12 +920,14 @@ def linear(x, weight: torch.Tensor, bias: Optional[torch.Tensor] = None,
     return out
 
 
-def linear_swiglu(x, gate_up_weight: torch.Tensor, activation: str = "silu") -> torch.Tensor:
+def linear_swiglu(x, gate_up_weight: torch.Tensor, activation: str = "silu",
+                  bounded: Optional[Tuple[float, float, float]] = None) -> torch.Tensor:
     """``act(x Wg^T) * (x Wu^T)`` for ``gate_up_weight = [Wg; Wu]`` of shape ``[2I, K]``
     and at most 16 rows of bfloat16 ``x`` (or a ``NormedRows``): the gate is applied to
     the 32-bit accumulators, the ``[M, 2I]`` intermediate is never stored.  17 to
     ``ROWS64_SWIGLU_ROWS`` rows are taken as ``NormedRows`` only (``rows64_swiglu_fusable``),
-    and with ``silu`` only.  ``activation``: one of ``GATE_ACTIVATIONS``."""
+    and with ``silu`` only.  ``activation``: one of ``GATE_ACTIVATIONS``.  ``bounded = (limit,
+    alpha, up_offset)``: the unit of ``clamped_glu`` instead (at most 16 rows)."""
     if activation not in GATE_ACTIVATIONS:
         raise KernelError(f"activation must be one of {sorted(GATE_ACTIVATIONS)}, got {activation!r}")
     if len(x.shape) != 2 or gate_up_weight.dim() != 2 or gate_up_weight.shape[0] % 2 \
@@ -929,6 +939,7 @@ def linear_swiglu(x, gate_up_weight: torch.Tensor, activation: str = "silu") -> 
     _need(gate_up_weight, "gate_up_weight", torch.bfloat16)
     if M > NORMED_ROWS_MAX_ROWS:
         if not (isinstance(x, NormedRows) and x.dtype == torch.bfloat16 and activation == "silu"
+                and bounded is None
                 and rows64_swiglu_fusable(M, K)):
             raise KernelError(f"linear_swiglu takes a step of {M} rows only as rows awaiting "
                               f"their norm, up to {ROWS64_SWIGLU_ROWS} rows, got K={K}")
@@ -953,7 +964,9 @@ def linear_swiglu(x, gate_up_weight: torch.Tensor, activation: str = "silu") -> 
         _ptr(normed.rows) if normed is not None else None,
         _ptr(normed.weight) if normed is not None else None,
         normed.eps if normed is not None else 0.0,
-        _ptr(gate_up_weight), _ptr(out), M, I, K, GATE_ACTIVATIONS[activation], _stream())
+        _ptr(gate_up_weight), _ptr(out), M, I, K,
+        GATE_ACTIVATIONS[activation] if bounded is None else BOUNDED_UNIT,
+        *(tuple(float(v) for v in bounded) if bounded is not None else (0.0, 0.0, 0.0)), _stream())
     _check(rc, "linear_swiglu", f"M={M} I={I} K={K}")
     _note("linear_swiglu", M=M, N=2 * I, K=K, norm_in_product=normed is not None)
     return out
@@ -1119,27 +1132,34 @@ class ScoreShape:
     and no value; None: none) and ``temperature`` (``(coef, every)``: the query at position
     ``p`` counts ``1 + coef * ln(floor((p + 1) / every) + 1)`` times; None: none); and to the
     mask, ``chunk``: positions are counted in chunks of that many from the sequence's start
-    and a query sees the earlier keys of its own chunk only (0: every earlier key)."""
+    and a query sees the earlier keys of its own chunk only (0: every earlier key), and
+    ``keep_first``: the first keys of the sequence, that many, count for every query behind them
+    whatever the window or the chunk (``paged_attention_gated`` and ``planes_attention``)."""
 
     def __init__(self, softcap: float = 0.0, sink: Optional[torch.Tensor] = None,
-                 temperature: Optional[Tuple[float, int]] = None, chunk: int = 0):
+                 temperature: Optional[Tuple[float, int]] = None, chunk: int = 0,
+                 keep_first: int = 0):
         self.softcap = float(softcap or 0.0)
         self.sink = sink
         self.chunk = int(chunk or 0)
-        if self.chunk < 0:
-            raise KernelError("a chunk must not be negative")
+        self.keep_first = int(keep_first or 0)
+        if self.chunk < 0 or self.keep_first < 0:
+            raise KernelError("a chunk and the number of kept keys must not be negative")
         self.coef, self.every = (float(temperature[0]), int(temperature[1])) if temperature \
             else (0.0, 0)
         if self.softcap < 0.0 or self.every < 0:
             raise KernelError("softcap and the temperature's period must not be negative")
 
-    def args(self, num_heads: int):
+    def args(self, num_heads: int, keeps: bool = False):
+        if self.keep_first and not keeps:
+            raise KernelError("this attention kernel knows no kept first keys")
         if self.sink is not None:
             _need(self.sink, "sink", torch.float32, (num_heads,))
         return self.softcap, _ptr(self.sink), self.coef, self.every, self.chunk
 
     def __bool__(self) -> bool:
-        return bool(self.softcap or self.sink is not None or self.every or self.chunk)
+        return bool(self.softcap or self.sink is not None or self.every or self.chunk
+                    or self.keep_first)
 
 
 def paged_attention(q: torch.Tensor, kv_cache: torch.Tensor, block_table: torch.Tensor,
@@ -1509,6 +1529,7 @@ def swiglu(gate_up: torch.Tensor) -> torch.Tensor:
 
 
 GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}
+BOUNDED_UNIT = 2        # the form of ``clamped_glu`` in the products that apply the gate themselves
 
 
 def gated_unit(gate_up: torch.Tensor, activation: str) -> torch.Tensor:
@@ -1737,13 +1758,20 @@ def qk_norm_rope_kv_write_wide(qkv: torch.Tensor, positions: torch.Tensor,
                                key_plane: Optional[torch.Tensor], value_plane: Optional[torch.Tensor],
                                num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int,
                                rotary_dim: int, adjacent_pairs: bool, eps: float,
-                               write_kv: bool = True) -> torch.Tensor:
+                               write_kv: bool = True, magnitude: float = 1.0,
+                               row_norm: Optional[Tuple[int, int]] = None) -> torch.Tensor:
     """As ``qk_norm_rope_kv_write`` for rows ``qkv [T, >= nh*d + nkv*d + nkv*dv]`` (further
     columns are left alone) and a cache whose pages hold a plane of keys
     ``[pages, kv_heads, page_size, head_dim]`` followed by a plane of values
     ``[pages, kv_heads, page_size, value_dim]`` (stored turned round, ``[value_dim][offset]``).
+    ``magnitude``: factor on cosine and sine.  ``num_kv_heads`` 0: rows of queries only, nothing
+    is stored.  ``row_norm = (q_count, k_count)``: one norm over all of a token's queries and one
+    over all of its keys, weights of ``num_heads * head_dim`` and ``num_kv_heads * head_dim``
+    elements, the means taken over that many elements.
     Returns the queries ``[T, num_heads, head_dim]``."""
     T, stride = qkv.shape
+    if num_kv_heads == 0 and write_kv:
+        raise KernelError("rows of queries only hold nothing to store")
     need = (num_heads + num_kv_heads) * head_dim + num_kv_heads * value_dim
     _need(qkv, "qkv", (torch.float32, torch.bfloat16))
     if stride < need:
@@ -1753,9 +1781,9 @@ def qk_norm_rope_kv_write_wide(qkv: torch.Tensor, positions: torch.Tensor,
         raise KernelError("head widths beyond 256 exceed the kernel's limit")
     if rotary_dim % 2 or not 0 <= rotary_dim <= head_dim:
         raise KernelError(f"rotary_dim {rotary_dim} must be even and at most head_dim {head_dim}")
-    for name, w in (("q_norm_w", q_norm_w), ("k_norm_w", k_norm_w)):
+    for name, w, heads in (("q_norm_w", q_norm_w, num_heads), ("k_norm_w", k_norm_w, num_kv_heads)):
         if w is not None:
-            _need(w, name, torch.float32, (head_dim,))
+            _need(w, name, torch.float32, (heads * head_dim if row_norm else head_dim,))
     if rotary_dim:
         _need(inv_freq, "inv_freq", torch.float32, (rotary_dim // 2,))
     page_size = 0
@@ -1766,12 +1794,24 @@ def qk_norm_rope_kv_write_wide(qkv: torch.Tensor, positions: torch.Tensor,
         page_size = _check_planes(key_plane, value_plane, qkv.dtype, num_kv_heads, head_dim,
                                   value_dim)
     q_out = torch.empty((T, num_heads, head_dim), dtype=qkv.dtype, device=qkv.device)
+    if row_norm:
+        if q_norm_w is None or write_kv and k_norm_w is None:
+            raise KernelError("a norm over the whole row needs its weights")
+        rc = _fn("rope_kv", "za_qk_row_norm_rope_kv_write")(
+            _ptr(qkv), _ptr(positions), _ptr(slots) if write_kv else None, _ptr(q_norm_w),
+            _ptr(k_norm_w), _ptr(inv_freq) if rotary_dim else None, _ptr(q_out),
+            _ptr(key_plane) if write_kv else None, _code(qkv.dtype), T, num_heads, num_kv_heads,
+            head_dim, value_dim, stride, rotary_dim, 1 if adjacent_pairs else 0, float(eps),
+            float(row_norm[0]), float(row_norm[1]), float(magnitude), page_size,
+            1 if write_kv else 0, _stream())
+        _check(rc, "qk_row_norm_rope_kv_write", f"heads {num_heads}+{num_kv_heads} of {head_dim}")
+        return q_out
     rc = _fn("rope_kv", "za_qk_norm_rope_kv_write_wide")(
         _ptr(qkv), _ptr(positions), _ptr(slots) if write_kv else None, _ptr(q_norm_w),
         _ptr(k_norm_w), _ptr(inv_freq) if rotary_dim else None, _ptr(q_out),
         _ptr(key_plane) if write_kv else None, _code(qkv.dtype), T, num_heads, num_kv_heads,
         head_dim, value_dim, stride, rotary_dim, 1 if adjacent_pairs else 0, float(eps),
-        page_size, 1 if write_kv else 0, _stream())
+        page_size, 1 if write_kv else 0, float(magnitude), _stream())
     _check(rc, "qk_norm_rope_kv_write_wide")
     return q_out
 
@@ -1847,7 +1887,7 @@ def paged_attention_gated(q: torch.Tensor, key_plane: torch.Tensor, value_plane:
             raise KernelError("keys_per_split must be a positive multiple of 64")
         part_acc = torch.empty((T, nh, nsplit, dv), dtype=torch.float32, device=q.device)
         part_ml = torch.empty((T, nh, nsplit, 2), dtype=torch.float32, device=q.device)
-    extras = shape.args(nh) if shape else (0.0, None, 0.0, 0, 0)
+    extras = shape.args(nh, keeps=True) + (shape.keep_first,) if shape else (0.0, None, 0.0, 0, 0, 0)
     rc = _fn("attention", "za_paged_attention_general")(
         _ptr(q), _ptr(out), _ptr(key_plane), _ptr(block_table), block_table.shape[1],
         _ptr(positions), _ptr(item_seq), _ptr(item_row0), _ptr(item_count), n_items, T,
@@ -1856,6 +1896,80 @@ def paged_attention_gated(q: torch.Tensor, key_plane: torch.Tensor, value_plane:
         int(gate_col), 1 if gate_element else 0, float(out_scale), *extras, _stream())
     _check(rc, "paged_attention_gated")
     _note("attention", kernel="plain", rows=T, dtype=q.dtype, nsplit=int(nsplit))
+    return out
+
+
+PLANES_TILE_KEYS = 64
+PLANES_ROWS = 128               # rows (token, head) of a work item
+PLANES_DECODE_GROUP = 16        # query heads a key/value head of the kernel for single tokens
+
+
+def planes_attention_supported(dtype: torch.dtype, num_heads: int, num_kv_heads: int, head_dim: int,
+                               value_dim: int, page_size: int = 4, scale: float = 1.0,
+                               shape: Optional[ScoreShape] = None) -> bool:
+    """Whether ``planes_attention`` takes these sizes and what ``shape`` asks for."""
+    return (dtype == torch.bfloat16 and head_dim % 8 == 0 and value_dim % 8 == 0
+            and head_dim <= 256 and value_dim <= 256 and page_size % 4 == 0 and scale > 0.0
+            and num_heads // num_kv_heads <= PLANES_ROWS
+            and not (shape is not None and (shape.softcap or shape.every)))
+
+
+def planes_attention(q: torch.Tensor, key_plane: torch.Tensor, value_plane: torch.Tensor,
+                     block_table: torch.Tensor, positions: torch.Tensor,
+                     items: Optional[Tuple[torch.Tensor, torch.Tensor, torch.Tensor, int]],
+                     scale: float, window: int = 0, tiles_per_split: int = 0, nsplit: int = 1,
+                     shape: Optional[ScoreShape] = None) -> torch.Tensor:
+    """Attention on the matrix cores over a plane of keys and a plane of values of any widths;
+    see csrc/attention_planes.hip.  ``q [T, heads, head_dim]`` bfloat16; returns ``[T, heads,
+    value_dim]``.  ``items``: work items ``(request, first row, rows, number)`` of at most
+    ``PLANES_ROWS // (heads // kv_heads)`` tokens, or ``None`` when every request brings one token
+    (at most ``PLANES_DECODE_GROUP`` query heads a key/value head).  An item's tiles of
+    ``PLANES_TILE_KEYS`` keys may be cut into ``nsplit`` ranges of ``tiles_per_split`` tiles.
+    ``shape``: its sink, chunk and kept first keys."""
+    if q.dim() != 3:
+        raise KernelError(f"q must be [T, heads, head_dim], got {tuple(q.shape)}")
+    T, nh, d = q.shape
+    _need(q, "q", torch.bfloat16)
+    nkv, dv = key_plane.shape[1], value_plane.shape[3]
+    page_size = _check_planes(key_plane, value_plane, q.dtype, nkv, d, dv)
+    if nh % nkv or not planes_attention_supported(q.dtype, nh, nkv, d, dv, page_size, scale, shape) \
+            or window < 0 or items is None and nh // nkv > PLANES_DECODE_GROUP:
+        raise KernelError(f"planes_attention does not take {nh} heads, {nkv} key/value heads, widths "
+                          f"{d} and {dv}, page size {page_size}, scale {scale}, window {window}")
+    _need(block_table, "block_table", torch.int32)
+    if block_table.dim() != 2:
+        raise KernelError("block_table must be [requests, max_pages]")
+    _need(positions, "positions", torch.int32, (T,))
+    if items is None:
+        if block_table.shape[0] < T:
+            raise KernelError("without work items every request brings exactly one token")
+        item_seq = item_row0 = item_count = None
+        n_items = T
+    else:
+        item_seq, item_row0, item_count, n_items = items
+        for name, t in (("item_seq", item_seq), ("item_row0", item_row0), ("item_count", item_count)):
+            _need(t, name, torch.int32)
+            if t.numel() < n_items:
+                raise KernelError(f"{name} holds {t.numel()} entries, fewer than {n_items} items")
+    out = torch.empty((T, nh, dv), dtype=q.dtype, device=q.device)
+    part_acc = part_ml = None
+    if nsplit > 1:
+        if tiles_per_split <= 0:
+            raise KernelError("tiles_per_split must be positive")
+        part_acc = torch.empty((T, nh, nsplit, dv), dtype=torch.float32, device=q.device)
+        part_ml = torch.empty((T, nh, nsplit, 2), dtype=torch.float32, device=q.device)
+    sink = shape.sink if shape is not None else None
+    if sink is not None:
+        _need(sink, "sink", torch.float32, (nh,))
+    rc = _fn("attention_planes", "za_planes_attention")(
+        _ptr(q), _ptr(out), _ptr(key_plane), _ptr(block_table), block_table.shape[1],
+        _ptr(positions), _ptr(item_seq), _ptr(item_row0), _ptr(item_count), n_items, T,
+        _ptr(part_acc), _ptr(part_ml), nh, nkv, d, dv, page_size, float(scale), int(window),
+        shape.keep_first if shape is not None else 0, shape.chunk if shape is not None else 0,
+        int(tiles_per_split), int(nsplit), _ptr(sink), _stream())
+    _check(rc, "planes_attention", f"heads {nh}/{nkv} widths {d}/{dv}")
+    _note("attention", kernel="planes" if items is not None else "planes_decode", rows=T,
+          dtype=q.dtype, nsplit=int(nsplit))
     return out
 
 

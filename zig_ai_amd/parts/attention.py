@@ -41,6 +41,16 @@ state).  These go through the path that takes the cache as two planes: the matri
 kernels where the sizes fit (the gate then is a small kernel behind them), the general
 attention kernel otherwise.
 
+Also on that path: ``qk_norm="row"`` (one RMS norm over all heads of a token's queries and one
+over all of its keys, weights as long as the projections), ``keep_first`` (with ``window``: the
+first so many keys of the sequence count for every query behind them; their pages stay when the
+window moves on), a position encoding with a ``magnitude``, and ``makes_kv=False`` (no key and
+value projections: the layer reads another layer's keys and values through its run-order
+entry, with queries, window and sink of its own).  Layers that share a cache entry name what
+it must hold for all of them, ``cache_window`` and ``cache_keep_first`` (by default the layer's
+own).  In bfloat16 these run on the matrix cores (``ops.planes_attention``: any widths, windows
+with kept keys, chunks, sinks).
+
 Head widths that are no multiple of 8 (what the kernels read at a time) are filled up with
 zeros when the part is built: zero rows of the q, k and v projections (and of their biases and
 filters), zero columns of the output projection; a score and a weighted sum do not change.
@@ -146,8 +156,11 @@ class GroupedQueryAttention(Mixer):
                  "k_proj.weight": TensorRule(((nkv * d, H),)),
                  "v_proj.weight": TensorRule(((nkv * dv, H),)),
                  "out_proj.weight": TensorRule(((H, nh * dv),))}
-        if params.get("values") == "keys":
+        own = bool(params.get("makes_kv", True))
+        if params.get("values") == "keys" or not own:
             del rules["v_proj.weight"]
+        if not own:
+            del rules["k_proj.weight"]
         if params.get("sink"):
             rules["sink"] = TensorRule(((nh,),), role="bias")
         if params.get("gate") == "head":
@@ -160,8 +173,10 @@ class GroupedQueryAttention(Mixer):
             rules["k_conv.weight"] = TensorRule(((nkv * d, taps),), role="filter")
             rules["v_conv.weight"] = TensorRule(((nkv * dv, taps),), role="filter")
         if params.get("qk_norm"):
-            rules["q_norm.weight"] = TensorRule(((d,),), role="norm")
-            rules["k_norm.weight"] = TensorRule(((d,),), role="norm")
+            row = params["qk_norm"] == "row"
+            rules["q_norm.weight"] = TensorRule(((nh * d if row else d,),), role="norm")
+            if own:
+                rules["k_norm.weight"] = TensorRule(((nkv * d if row else d,),), role="norm")
         if params.get("bias"):
             rules["q_proj.bias"] = TensorRule(((nh * d,),), role="bias")
             rules["k_proj.bias"] = TensorRule(((nkv * d,),), role="bias")
@@ -176,10 +191,10 @@ class GroupedQueryAttention(Mixer):
         nkv *= _kv_repeat(int(params["num_heads"]), nkv)    # (as they lie in the cache)
         dv = _round_up8(params.get("value_dim") or d)       # (filled up)
         d = _round_up8(d)
-        if dv == d:
-            paged = PagedNeed.kv(nkv, d, int(params.get("window") or 0))
-        else:
-            paged = PagedNeed(((nkv, d), (nkv, dv)), int(params.get("window") or 0))
+        # (what the entry holds for every layer that reads it)
+        window = int(params.get("cache_window", params.get("window")) or 0)
+        keep = int(params.get("cache_keep_first", params.get("keep_first")) or 0) if window else 0
+        paged = PagedNeed(((nkv, d), (nkv, dv)), window, keep_first=keep)
         taps = int(params.get("conv") or 0)
         if not taps:
             return paged
@@ -199,6 +214,13 @@ class GroupedQueryAttention(Mixer):
         self.model_value_dim = int(params.get("value_dim") or self.model_head_dim)
         self.head_dim, self.value_dim = _round_up8(self.model_head_dim), _round_up8(self.model_value_dim)
         norm_eps = float(params.get("norm_eps", 0.0))
+        self.makes_kv = bool(params.get("makes_kv", True))
+        if params.get("qk_norm") not in (None, False, True, "row"):
+            raise ValueError(f"qk_norm must be true, false or 'row', got {params.get('qk_norm')!r}")
+        # one norm over all heads: (elements of the queries', of the keys') mean
+        self.row_norm = (self.num_heads * self.model_head_dim,
+                         self.num_kv_heads * self.model_head_dim) \
+            if params.get("qk_norm") == "row" else None
         if (self.head_dim, self.value_dim) != (self.model_head_dim, self.model_value_dim):
             tensors, norm_eps = self._filled_up(params, tensors, norm_eps)
         repeat = _kv_repeat(self.num_heads, self.num_kv_heads)
@@ -208,6 +230,10 @@ class GroupedQueryAttention(Mixer):
                          "v_proj.bias", "v_conv.weight"):
                 if name in tensors:
                     tensors[name] = _repeat_heads(tensors[name], self.num_kv_heads, repeat)
+            if self.row_norm and self.makes_kv:
+                tensors["k_norm.weight"] = _repeat_heads(tensors["k_norm.weight"],
+                                                         self.num_kv_heads, repeat)
+                self.row_norm = (self.row_norm[0], self.row_norm[1] * repeat)
             self.num_kv_heads *= repeat
             self.group //= repeat
         if params.get("gate") not in (None, "head", "element"):
@@ -220,10 +246,24 @@ class GroupedQueryAttention(Mixer):
         if self.chunk < 0 or self.taps < 0 or self.taps > ops.CONV_MAX_TAPS:
             raise ValueError(f"chunk {self.chunk} and conv {self.taps}: neither negative, at most "
                              f"{ops.CONV_MAX_TAPS} taps")
-        # values of their own width, a gate, chunks or a convolution: the kernels that take
+        self.window = int(params.get("window") or 0)
+        self.keep_first = int(params.get("keep_first") or 0) if self.window else 0
+        if self.window < 0 or self.keep_first < 0:
+            raise ValueError(f"window {self.window} and keep_first {self.keep_first}: neither may be "
+                             f"negative")
+        pos = params.get("position")
+        self.position = None
+        if pos is not None:
+            self.position = lookup("position", pos.kind)(pos.params, {}, runtime)
+        self.magnitude = float(getattr(self.position, "magnitude", 1.0))
+        # values of their own width, a gate, chunks, a convolution, ...: the kernels that take
         # the cache as two planes
         self.wide = self.gated or self.value_dim != self.head_dim or bool(self.chunk) \
-            or bool(self.taps) or params.get("sink_value") is not None
+            or bool(self.taps) or params.get("sink_value") is not None or self.row_norm is not None \
+            or self.keep_first > 0 or self.magnitude != 1.0 or not self.makes_kv
+        if not self.makes_kv and (self.taps or params.get("bias") or params.get("values") == "keys"):
+            raise ValueError("a layer without keys and values of its own takes no convolution, no "
+                             "bias and no values that are its keys")
         if self.value_dim % 8 or self.value_dim > 256:
             raise ValueError(f"value_dim {self.value_dim} must be a multiple of 8, at most 256")
         if self.group > ops.ATTENTION_MAX_ROWS:
@@ -237,7 +277,6 @@ class GroupedQueryAttention(Mixer):
         self.rows_per_item = max(1, ops.ATTENTION_MAX_ROWS // self.group)
         self.mfma_rows_per_item = max(1, ops.ATTENTION_MFMA_ROWS // self.group)
         self.mfma_decode_rows_per_item = max(1, ops.ATTENTION_MFMA_DECODE_ROWS // self.group)
-        self.window = int(params.get("window") or 0)
         scale = params.get("softmax_scale")
         self.scale = float(scale) if scale is not None else 1.0 / math.sqrt(self.model_head_dim)
         # whether the matrix-core kernels take these sizes (the page size is checked per step)
@@ -260,11 +299,13 @@ class GroupedQueryAttention(Mixer):
             sink = torch.full((self.num_heads,), float(params["sink_value"]), dtype=torch.float32,
                               device=runtime.device)
         self.shape = ops.ScoreShape(params.get("softcap") or 0.0, sink,
-                                    tuple(temperature) if temperature else None, self.chunk)
-        opening = [tensors["q_proj.weight"], tensors["k_proj.weight"],
-                   tensors["k_proj.weight" if self.shared_values else "v_proj.weight"]]
-        self.gate_col = (self.num_heads + self.num_kv_heads) * self.head_dim \
-            + self.num_kv_heads * self.value_dim
+                                    tuple(temperature) if temperature else None, self.chunk,
+                                    self.keep_first)
+        opening = [tensors["q_proj.weight"]]
+        if self.makes_kv:
+            opening += [tensors["k_proj.weight"],
+                        tensors["k_proj.weight" if self.shared_values else "v_proj.weight"]]
+        self.gate_col = sum(w.shape[0] for w in opening)
         if self.gated:
             opening.append(tensors["gate_proj.weight"])
         self.w_qkv = fuse_rows(*opening)
@@ -286,10 +327,6 @@ class GroupedQueryAttention(Mixer):
                                      tensors["v_conv.weight"]], dim=0).contiguous()
         self.q_norm = tensors.get("q_norm.weight") if params.get("qk_norm") else None
         self.k_norm = tensors.get("k_norm.weight") if params.get("qk_norm") else None
-        pos = params.get("position")
-        self.position = None
-        if pos is not None:
-            self.position = lookup("position", pos.kind)(pos.params, {}, runtime).without_magnitude()
         self.fused_rotation = bool(getattr(self.position, "fused_rotation", False))
         # recorded into a graph only if the position encoding, too, never looks at a
         # step's numbers on the host
@@ -298,9 +335,19 @@ class GroupedQueryAttention(Mixer):
         if self.wide and self.position is not None and not self.fused_rotation:
             raise ValueError("an attention with value_dim or gate takes a rotary position "
                              "encoding or none")
-        self.mfma = self.mfma and self.value_dim == self.head_dim
+        self.mfma = self.mfma and self.value_dim == self.head_dim and not self.keep_first
+        # the matrix-core kernels for planes of any widths
+        self.planes = self.wide and not self.mfma and not self.gated and not self.taps \
+            and ops.planes_attention_supported(runtime.dtype, self.num_heads, self.num_kv_heads,
+                                               self.head_dim, self.value_dim, scale=self.scale,
+                                               shape=self.shape)
+        if self.planes:
+            self.kernel_sources = type(self).kernel_sources + ("attention_planes",)
+        self.planes_rows_per_item = max(1, ops.PLANES_ROWS // self.group)
         if not self.mfma:
-            self.item_granularities = [self.rows_per_item]
+            # (the general kernel takes the pages that the matrix-core kernels do not)
+            self.item_granularities = [self.rows_per_item] + (
+                [self.planes_rows_per_item] if self.planes else [])
         self.rotation_in_attention = (
             not self.wide and self.fused_rotation and runtime.dtype == torch.bfloat16
             and self.position.rotary_dim == self.head_dim and self.position.pairing != "adjacent")
@@ -310,7 +357,7 @@ class GroupedQueryAttention(Mixer):
     def _filled_up(self, params, tensors, eps: float):
         """The part's tensors with every head filled up with zeros to the kernels' widths, and
         the eps that goes with the padded per-head norm."""
-        nh, nkv = self.num_heads, self.num_kv_heads
+        nh, nkv, row = self.num_heads, self.num_kv_heads, self.row_norm is not None
         d0, dv0, d, dv = self.model_head_dim, self.model_value_dim, self.head_dim, self.value_dim
         t = dict(tensors)
         for name, heads, w0, w1 in (("q", nh, d0, d), ("k", nkv, d0, d), ("v", nkv, dv0, dv)):
@@ -321,8 +368,15 @@ class GroupedQueryAttention(Mixer):
             t["gate_proj.weight"] = _pad_heads(t["gate_proj.weight"], nh, dv0, dv)
         t["out_proj.weight"] = _pad_heads(t["out_proj.weight"].t().contiguous(), nh, dv0, dv) \
             .t().contiguous()
-        if params.get("qk_norm"):
+        if row:
+            # (the mean is taken over the model's elements, whatever the row's length)
+            for name, heads in (("q_norm.weight", nh), ("k_norm.weight", nkv)):
+                if name in t:
+                    t[name] = _pad_heads(t[name], heads, d0, d)
+        elif params.get("qk_norm"):
             for name in ("q_norm.weight", "k_norm.weight"):
+                if name not in t:
+                    continue
                 w = t[name].float() * math.sqrt(d0 / d)
                 t[name] = torch.cat([w, w.new_zeros((d - d0,))]).contiguous()
             eps = eps * d0 / d
@@ -421,6 +475,9 @@ class GroupedQueryAttention(Mixer):
         q | k | v | gate, the cache a plane of keys and a plane of values."""
         nh, nkv, d, dv = self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim
         T = x.shape[0]
+        if cache.writes and not self.makes_kv:
+            raise ValueError("an attention without keys and values of its own reads another layer's "
+                             "cache: its run-order entry must not write")
         qkv = ops.linear(x, self.w_qkv, self.b_qkv, tune=self.runtime.tune)
         key_plane, value_plane = cache.planes
         rot = self.position.rotary_dim if self.position is not None else 0
@@ -433,8 +490,10 @@ class GroupedQueryAttention(Mixer):
                                   out_dtype=qkv.dtype)
         q = ops.qk_norm_rope_kv_write_wide(
             qkv, step.positions, step.slot_mapping[cache.group], self.q_norm, self.k_norm,
-            self.position.inv_freq if rot else None, key_plane, value_plane, nh, nkv, d, dv, rot,
-            bool(rot) and self.position.pairing == "adjacent", self.eps, write_kv=cache.writes)
+            self.position.inv_freq if rot else None, key_plane, value_plane, nh,
+            nkv if self.makes_kv else 0, d, dv, rot,
+            bool(rot) and self.position.pairing == "adjacent", self.eps, write_kv=cache.writes,
+            magnitude=self.magnitude, row_norm=self.row_norm)
         table = step.block_tables[cache.group]
         # (ranges are cut at absolute key positions: behind a window nearly all of them
         # would be empty, so a windowed layer's contexts are never cut)
@@ -456,6 +515,16 @@ class GroupedQueryAttention(Mixer):
                                                     self.window, keys, nsplit, shape=self.shape)
             if gate is not None:
                 ops.head_gate_(o, gate, self.gate_col, element=self.gate_element)
+        elif self.planes and key_plane.shape[2] % 4 == 0:
+            items = None
+            if step.n_tokens > step.n_seqs or self.group > ops.PLANES_DECODE_GROUP:
+                items = step.attention_items(self.planes_rows_per_item)
+            # (an item's list of tiles is cut, not the context: behind a window it stays short)
+            tiles, nsplit = self._plan_tiles(items[3] if items else step.n_seqs,
+                                             self._reach(step.max_keys),
+                                             SPLIT_TARGET if items is None else BUSY_WORKGROUPS)
+            o = ops.planes_attention(q, key_plane, value_plane, table, step.positions, items,
+                                     self.scale, self.window, tiles, nsplit, shape=self.shape)
         else:
             item_seq, item_row0, item_count, n_items = step.attention_items(self.rows_per_item)
             keys, nsplit = split(n_items)
@@ -467,7 +536,19 @@ class GroupedQueryAttention(Mixer):
             step.taps["q"] = q.clone()
             step.taps["o"] = o.clone()
         return ops.linear(o.view(T, nh * dv), self.w_out, self.b_out, accumulate=stream,
-                          tune=self.runtime.tune)
+                          partial_ok=self.partial_ok, tune=self.runtime.tune)
+
+    def _reach(self, max_keys: int) -> int:
+        """About how many keys a query sees of a context of ``max_keys``."""
+        for limit in (self.window, self.chunk):
+            if limit:
+                max_keys = min(max_keys, limit + self.keep_first)
+        return max_keys
+
+    def _plan_tiles(self, n_items: int, keys: int, target: int):
+        """``plan_split`` in tiles of the kernel."""
+        per_range, nsplit = plan_split(n_items, self.num_kv_heads, keys, target=target)
+        return -(-per_range // ops.PLANES_TILE_KEYS), nsplit
 
     def _leave_taps(self, step, cache, q: torch.Tensor, o: torch.Tensor) -> None:
         """Diagnostics: the queries, the keys and values of the step's tokens as they lie in

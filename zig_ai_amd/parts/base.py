@@ -58,19 +58,21 @@ class PagedNeed:
     vectors of ``width`` elements per token.  Keys and values are two planes of
     ``(num_kv_heads, head_dim)`` (``PagedNeed.kv``); a mixer that keeps one latent
     vector per token has one plane ``(1, width)``; planes may differ in size.  With
-    ``window > 0`` only the last ``window`` positions are ever read, so older pages
-    can be given back.  ``dtype``: what the planes store (``None``: the run's storage
+    ``window > 0`` only the last ``window`` positions are ever read, and the first
+    ``keep_first`` positions of the sequence, so the pages between can be given back.
+    ``dtype``: what the planes store (``None``: the run's storage
     type)."""
 
     planes: Tuple[Tuple[int, int], ...]
     window: int = 0
     dtype: Optional[torch.dtype] = None
+    keep_first: int = 0
 
     @classmethod
     def kv(cls, num_kv_heads: int, head_dim: int, window: int = 0,
-           dtype: Optional[torch.dtype] = None) -> "PagedNeed":
+           dtype: Optional[torch.dtype] = None, keep_first: int = 0) -> "PagedNeed":
         plane = (int(num_kv_heads), int(head_dim))
-        return cls((plane, plane), int(window), dtype)
+        return cls((plane, plane), int(window), dtype, int(keep_first))
 
     @property
     def is_kv(self) -> bool:

@@ -104,7 +104,8 @@ class ClampedGLU(FeedForward):
         y = (g * sigmoid(alpha * g) * (u + up_offset)) Wd^T
 
     ``limit`` (none if 0), ``alpha`` and ``up_offset`` come from ``params``.  Gate and up
-    weights are one matrix, as in ``SwiGLU``; the activation is a kernel of its own."""
+    weights are one matrix, as in ``SwiGLU``.  In a decode batch the product applies the unit to
+    its own sums, otherwise the unit is a kernel of its own."""
 
     kind = "clamped_glu"
     graph_safe = True
@@ -125,9 +126,13 @@ class ClampedGLU(FeedForward):
         self.down = ops.projection_weight(tensors["down.weight"])
 
     def forward(self, x, step=None):
-        a = ops.clamped_glu(ops.linear(x, self.gate_up, tune=self.runtime.tune), self.limit,
-                            self.alpha, self.up_offset)
-        return ops.linear(a, self.down, tune=self.runtime.tune)
+        if x.dtype == torch.bfloat16 and self.gate_up.dtype == torch.bfloat16 \
+                and x.shape[0] <= 16 and x.shape[1] <= 8192:
+            a = ops.linear_swiglu(x, self.gate_up, bounded=(self.limit, self.alpha, self.up_offset))
+        else:
+            a = ops.clamped_glu(ops.linear(x, self.gate_up, tune=self.runtime.tune), self.limit,
+                                self.alpha, self.up_offset)
+        return ops.linear(a, self.down, partial_ok=self.partial_ok, tune=self.runtime.tune)
 
 
 class ActivatedMLP(FeedForward):
