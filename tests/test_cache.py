@@ -166,6 +166,29 @@ def test_reserve_is_all_or_nothing():
     m.check()
 
 
+@pytest.mark.parametrize("keep,pages_kept", [(0, 0), (1, 1), (4, 1), (5, 2), (40, 10)])
+def test_kept_first_tokens_keep_their_pages(keep, pages_kept):
+    """Behind a window every page goes back but those with the sequence's first tokens."""
+    need = PagedNeed(((2, 16), (2, 8)), 6, keep_first=keep)
+    m = CacheManager({0: need, 1: PagedNeed(((2, 16), (2, 8)), 6)}, 4, 20, 2, allocate=False)
+    assert len(m.groups) == (2 if keep else 1)         # kept tokens make a group of their own
+    for name in ("a", "b"):
+        m.admit(name)
+        for n in (3, 9, 1, 1, 1, 14, 1, 1):            # 31 tokens: the window starts at 26
+            m.reserve(name, n)
+            m.commit(name, n)
+            m.check()
+        table = m.table(name, 0)
+        assert len(table) == 8
+        held = [p for p, page in enumerate(table) if page != FREED]
+        assert held == sorted(set(range(min(pages_kept, 8))) | {6, 7})
+        m.release(name)
+        m.check()
+    assert m.groups[0].pool.free_count == 20
+    with pytest.raises(ValueError):
+        CacheManager({0: PagedNeed(((2, 16),), 6, keep_first=-1)}, 4, 4, 1, allocate=False)
+
+
 def test_window_gives_pages_back():
     m = manager(num_pages=8, page_size=4, window=6)
     m.admit("r")
