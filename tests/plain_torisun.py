@@ -111,8 +111,10 @@ def attention(h: torch.Tensor, tensors, p: str, m: Mapping, eps: float,
 
 # ----------------------------------------------------------------- feed-forward
 def dense(h: torch.Tensor, tensors, p: str, limit: float) -> torch.Tensor:
-    g = (h @ _w(tensors, p + "gate").T).clamp(max=limit)
-    u = (h @ _w(tensors, p + "up").T).clamp(-limit, limit)
+    """``limit`` 0: no bounds."""
+    g, u = h @ _w(tensors, p + "gate").T, h @ _w(tensors, p + "up").T
+    if limit:
+        g, u = g.clamp(max=limit), u.clamp(-limit, limit)
     return (g * torch.sigmoid(1.702 * g) * (u + 1.0)) @ _w(tensors, p + "down").T
 
 
@@ -156,7 +158,7 @@ def forward(config: Mapping, tensors: Mapping[str, torch.Tensor], token_ids: Lis
                                None if source is None else made[int(source)])
         x = x + rms_norm(y, _w(tensors, p + "norm1"), eps)
         if mlp is not None:
-            y = dense(x, tensors, p + "mlp.", float(mlp["limit"])) if mlp["kind"] == "dense" \
+            y = dense(x, tensors, p + "mlp.", float(mlp.get("limit", 0.0))) if mlp["kind"] == "dense" \
                 else experts(x, tensors, p + "mlp.", mlp)
             x = x + rms_norm(y, _w(tensors, p + "norm2"), eps)
         if streams is not None:
