@@ -287,11 +287,33 @@ def vupelorn_shape(width, layers, vocab):
             "layers": out, "max_position_embeddings": 128000}
 
 
+def torisun_shape(width, layers, vocab):
+    """Layer sizes in the manner of a real model of this design: query heads of 128 elements, four a
+    key head, values of 64, windows of 1,024 tokens beside the first four, frequencies stretched
+    by 8; every other layer reads the keys and values of the one before it; a dense feed-forward
+    of four times the width and 32 experts of half the width (4 a token, one shared) in turn."""
+    heads = width // 128
+    own = {"heads": heads, "kv_heads": max(1, heads // 4), "dim": 128, "vdim": 64,
+           "scale": 128 ** -0.5, "mask": {"size": 1024, "keep_first": 4},
+           "rot": {"dims": 128, "base": 5e5, "scaling": {"factor": 8.0, "original": 4096,
+                                                         "fast": 32.0, "slow": 1.0}}}
+    dense = {"kind": "dense", "ff": 4 * width, "limit": 7.0}
+    moe = {"kind": "moe", "expert": {"ff": width // 2}, "shared": {"ff": width // 2},
+           "router": {"experts": 32, "top": 4, "scale": 2.5}}
+    out = []
+    for i in range(layers):
+        out.append({"type": "attention", "mixer": own if i % 2 == 0 else dict(own, kv_from=i - 1),
+                    "mlp": dense if i % 2 == 0 else moe})
+    return {"architecture": "Torisun", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+            "layers": out, "max_position_embeddings": 128000}
+
+
 def compare(widths, layers, batch, prompt_len, steps, warmup, design="rudilix", only=None) -> dict:
     """Prefill and decode throughput of Rudilix and of LFM2 at equal sizes, or
     (``design="ranesun"``) of Ranesun and of Rudilix, or (``design="gemodra"``) of Gemodra and
     of Ranesun, or (``design="nopozen"``) of Nopozen and of Ranesun, or
-    (``design="vupelorn"``) of Vupelorn, of Gemodra and of Nopozen."""
+    (``design="vupelorn"``) of Vupelorn, of Gemodra and of Nopozen, or (``design="torisun"``) of
+    Torisun, of Vupelorn and of Nopozen."""
     import torch
     from zig_ai_amd.engine import DecoderModel, ModelRunner, StepEntry
     from zig_ai_amd.kernels import ops
@@ -386,7 +408,9 @@ def compare(widths, layers, batch, prompt_len, steps, warmup, design="rudilix", 
                     "gemodra": {"gemodra": gemodra_shape, "ranesun": ranesun_shape},
                     "nopozen": {"nopozen": nopozen_shape, "ranesun": ranesun_shape},
                     "vupelorn": {"vupelorn": vupelorn_shape, "gemodra": gemodra_shape,
-                                 "nopozen": nopozen_shape}}[design]
+                                 "nopozen": nopozen_shape},
+                    "torisun": {"torisun": torisun_shape, "vupelorn": vupelorn_shape,
+                                "nopozen": nopozen_shape}}[design]
             result["widths"][str(width)] = {name: measure(shape(width, layers, vocab))
                                             for name, shape in pair.items()
                                             if only in (None, name)}
@@ -446,10 +470,12 @@ def main() -> int:
     ap.add_argument("--compare-widths", default="1024,2048",
                     help="--workload compare: the widths, with commas between them")
     ap.add_argument("--compare-layers", type=int, default=8, help="--workload compare: layers")
-    ap.add_argument("--compare-design", choices=["rudilix", "ranesun", "gemodra", "nopozen", "vupelorn"],
+    ap.add_argument("--compare-design", choices=["rudilix", "ranesun", "gemodra", "nopozen", "vupelorn",
+                                                      "torisun"],
                     default="rudilix",
                     help="--workload compare: rudilix (beside LFM2), ranesun (beside Rudilix), "
-                         "gemodra or nopozen (beside Ranesun), vupelorn (beside Gemodra and Nopozen)")
+                         "gemodra or nopozen (beside Ranesun), vupelorn (beside Gemodra and Nopozen), "
+                         "torisun (beside Vupelorn and Nopozen)")
     ap.add_argument("--compare-only", default=None,
                     help="--workload compare: measure this model of the pair alone (for a profiler)")
     ap.add_argument("--workload", choices=["steps", "serve", "compare"], default="steps",

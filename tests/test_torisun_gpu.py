@@ -769,3 +769,60 @@ def test_bounded_unit_in_the_product(M, I, K):
             a, u = a.clamp(max=limit), u.clamp(-limit, limit)
         want = a * torch.sigmoid(1.702 * a) * (u + 1.0)
         assert float((got - want).abs().max()) < 1e-2 * float(want.abs().max()), limit
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("width", [36, 256, 3000])
+def test_normed_rows_of_the_embedding(dtype, width):
+    from zig_ai_amd.kernels import ops
+    g = torch.Generator().manual_seed(width)
+    table = (torch.randn(19, width, generator=g) * 3).to(dtype)
+    w = torch.randn(width, generator=g)
+    ids = torch.randint(0, 19, (7,), generator=g, dtype=torch.int32)
+    want = plain.rms_norm(table[ids.long()].double(), w.double(), 1e-2)
+    rows, copy = ops.embed_norm(ids.cuda(), table.cuda(), w.cuda(), 1e-2, torch.bfloat16)
+    assert float((rows.cpu().double() - want).abs().max()) < 1e-5 * float(want.abs().max())
+    assert torch.equal(copy, rows.to(torch.bfloat16))
+    assert ops.embed_norm(ids.cuda(), table.cuda(), w.cuda(), 1e-2)[1] is None
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("E,top,N,K,T", [(5, 2, 24, 40, 3), (4, 3, 72, 64, 50), (3, 2, 200, 136, 300), (9, 1, 8, 24, 1)])
+def test_grouped_products_with_gates_and_weights(dtype, E, top, N, K, T):
+    """The gated unit on the product's own sums, weights an assignment ahead of it and behind
+    the plain product, results written as planes of a given stack: decode batches, tiles of 64
+    rows and tiles of 128."""
+    from zig_ai_amd.kernels import ops
+    dev = torch.device("cuda")
+    g = torch.Generator().manual_seed(E * N + T)
+    x = torch.randn(T, K, generator=g).to(dtype)
+    w = (torch.randn(E, 2 * N, K, generator=g) * 1.5 * K ** -0.5).to(dtype)
+    chosen = torch.stack([torch.randperm(E, generator=g)[:top] for _ in range(T)]).int()
+    weight = torch.rand(T, top, generator=g) + 0.2
+    lists, counts = ops.expert_lists(None, chosen.to(dev), T, E)
+    sums = torch.stack([w[chosen[t, j]].double() @ x[t].double() for t in range(T) for j in range(top)])
+    a, u = sums[:, :N], sums[:, N:]
+    tol = 1e-5 if dtype == torch.float32 else 1e-2
+    r = weight.reshape(-1, 1).double()
+    wants = {"silu": (a * torch.sigmoid(a) * u, dict(gate="silu")),
+             "gelu": (torch.nn.functional.gelu(a, approximate="tanh") * u, dict(gate="gelu_tanh")),
+             "bounded": ((lambda p, q: p * torch.sigmoid(1.7 * p) * (q + 0.5))(
+                 (r * a).clamp(max=0.8), (r * u).clamp(-0.8, 0.8)),
+                 dict(bounded=(0.8, 1.7, 0.5), row_weight=weight.to(dev)))}
+    for name, (want, kw) in wants.items():
+        for out_dtype in (dtype, torch.float32):
+            got = ops.grouped_linear(x.to(dev), w.to(dev), lists, counts, T, per_token=True,
+                                     out_dtype=out_dtype, **kw).cpu().double()
+            assert float((got - want).abs().max()) < tol * float(want.abs().max()), (name, out_dtype)
+    rows = torch.randn(T * top, K, generator=g).to(dtype)
+    want = torch.stack([r[i] * (w[chosen.reshape(-1)[i]].double() @ rows[i].double()) for i in range(T * top)])
+    stack = torch.full((top + 1, T, 2 * N), 7.0, dtype=torch.float32, device=dev)
+    ops.grouped_linear(rows.to(dev), w.to(dev), lists, counts, T, per_token=False, stacked=True,
+                       row_weight=weight.to(dev), out=stack[:top])
+    got = stack[:top].permute(1, 0, 2).reshape(T * top, 2 * N).cpu().double()
+    assert float((got - want).abs().max()) < tol * float(want.abs().max())
+    assert bool((stack[top] == 7.0).all())
+    # a plain product into the plane behind
+    ops.linear(x.to(dev), w[0].contiguous().to(dev), out_dtype=torch.float32, into=stack[top])
+    want = x.double() @ w[0].double().T
+    assert float((stack[top].cpu().double() - want).abs().max()) < tol * float(want.abs().max())

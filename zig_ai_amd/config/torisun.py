@@ -266,7 +266,8 @@ class TorisunConfig:
         if s.kind == "dense":
             return PartSpec("clamped_glu",
                             {"hidden_size": H, "intermediate_size": s.ff, "limit": s.limit,
-                             "alpha": GATE_SLOPE, "up_offset": UP_OFFSET},
+                             "alpha": GATE_SLOPE, "up_offset": UP_OFFSET,
+                             "unit_in_product": True},
                             {f"{w}.weight": (p + w,) for w in ("gate", "up", "down")})
         names = {"router.weight": (p + "router",)}
         for e in range(s.experts):

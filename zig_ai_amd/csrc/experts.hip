@@ -17,7 +17,11 @@
 //    assignment.  dst(a) = a, or, `stacked`, (a % top) * T + a / top: a stack [top][T][N]
 //    of 32-bit partial results, which the norm that follows adds up in its order (so the
 //    weighted sum over a token's experts is taken in 32-bit and costs no kernel).
-//    f: nothing, or the square of relu.
+//    f: nothing, or the square of relu; or, `gate`, the gated unit of two columns: W then has
+//    2N rows, gate rows ahead of up rows, and out[.., n] = act(v[n]) * v[N + n] from the 32-bit
+//    sums (a wave holds both columns), so the products' 2N columns are never stored.
+//    `row_weight`: one number an assignment, times the result, or with a gate times the sums
+//    ahead of it (a weight on an expert's input; there are no biases).
 //    How many tiles there are is known on the device only; the grid is the upper bound
 //    ceil(A / TM) + E and a workgroup beyond the last tile leaves at once.
 //    Every output element is a sum over k in an order fixed by K alone: a token's result
@@ -85,6 +89,9 @@ struct GroupedArgs {
   int A, T, top, E, N, K;
   int src_div, stacked, act;
   float out_scale;
+  const float* row_weight;   // [A] or null
+  int gate;                  // 0: none, 1: silu, 2: the tanh form of gelu, 3: bounded
+  float bound, slope, offset;
 };
 
 // The expert and the tile within it that workgroup `b` serves; false when there is none.
@@ -113,6 +120,23 @@ __device__ __forceinline__ float expert_act(float v, int act) {
   return v;
 }
 
+// The gated unit (gate > 0) of one assignment's sums `v` (gate) and `u` (up).
+__device__ __forceinline__ float expert_unit(const GroupedArgs& g, float v, float u, float w) {
+  v *= w;
+  u *= w;
+  if (g.gate == 3) {
+    if (g.bound > 0.f) {
+      v = fminf(v, g.bound);
+      u = fminf(fmaxf(u, -g.bound), g.bound);
+    }
+    return v * (1.0f / (1.0f + expf(-g.slope * v))) * (u + g.offset);
+  }
+  const float a = g.gate == 2
+                      ? 0.5f * v * (1.0f + tanhf(0.7978845608028654f * (v + 0.044715f * v * v * v)))
+                      : v * (1.0f / (1.0f + expf(-v)));
+  return a * u;
+}
+
 __device__ __forceinline__ size_t dst_row(const GroupedArgs& g, int a) {
   return g.stacked ? (size_t)(a % g.top) * g.T + a / g.top : (size_t)a;
 }
@@ -120,32 +144,34 @@ __device__ __forceinline__ size_t dst_row(const GroupedArgs& g, int a) {
 // Operand layout of v_mfma_f32_16x16x32_bf16: lane l supplies row (l % 16), k-slots
 // (l / 16) * 8 .. + 7 of either operand and receives rows (l / 16) * 4 .. + 3, column
 // (l % 16) of the product.
-template <int TM, typename TO>
+template <int TM, typename TO, bool GATED>
 __global__ void __launch_bounds__(256)
 grouped_gemm_bf16_kernel(GroupedArgs g) {
   constexpr int WM = TM / 16;          // waves along the rows
   constexpr int WN = 4 / WM;           // waves along the columns
-  constexpr int NT = 4 / WN;           // 16-column tiles a wave
+  // 16-column blocks of the output a wave, and its tiles of weight rows (gate and up in turn)
+  constexpr int NB = GATED ? (TM == 16 ? 1 : 2) : 4 / WN;
+  constexpr int NT = GATED ? 2 * NB : NB;
   int e, tile, count;
   if (!find_tile<TM>(g.counts, g.E, blockIdx.x, &e, &tile, &count)) return;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int wm = wave % WM, wn = wave / WM;
   const int r16 = lane & 15, kq = lane >> 4;
-  const int n0 = blockIdx.y * 64 + wn * NT * 16;
+  const int n0 = blockIdx.y * (WN * NB * 16) + wn * NB * 16;
   const int* mine = g.lists + (size_t)e * g.A;
   const int K = g.K, N = g.N;
 
   const int row = tile * TM + wm * 16 + r16;
   const bool row_ok = row < count;
   const bf16_t* arow = (const bf16_t*)g.src + (size_t)(row_ok ? mine[row] / g.src_div : 0) * K;
-  const bf16_t* wbase = (const bf16_t*)g.W + (size_t)e * N * K;
+  const bf16_t* wbase = (const bf16_t*)g.W + (size_t)e * (GATED ? 2 * N : N) * K;
   const bf16_t* wrow[NT];
   bool col_ok[NT];
 #pragma unroll
   for (int j = 0; j < NT; ++j) {
-    const int n = n0 + j * 16 + r16;
+    const int n = n0 + (GATED ? j / 2 : j) * 16 + r16;
     col_ok[j] = n < N;
-    wrow[j] = wbase + (size_t)(col_ok[j] ? n : 0) * K;
+    wrow[j] = wbase + (size_t)(col_ok[j] ? n + (GATED && (j & 1) ? N : 0) : 0) * K;
   }
   f32x4_t acc[NT];
 #pragma unroll
@@ -154,7 +180,7 @@ grouped_gemm_bf16_kernel(GroupedArgs g) {
 
   // steps of 32 at a time (two, or four where a wave has one column tile: a decode batch,
   // which only streams weights): their loads are all requested before the first product
-  constexpr int U = NT == 1 ? 4 : 2;
+  constexpr int U = NB == 1 ? 4 : 2;
   for (int k0 = 0; k0 < K; k0 += 32 * U) {
     bf16x8_t fa[U], fw[U][NT];
 #pragma unroll
@@ -179,10 +205,15 @@ grouped_gemm_bf16_kernel(GroupedArgs g) {
     const int r = tile * TM + wm * 16 + kq * 4 + i;
     if (r >= count) continue;
     const size_t d = dst_row(g, mine[r]);
+    const float w = g.row_weight ? g.row_weight[mine[r]] : 1.0f;
 #pragma unroll
-    for (int j = 0; j < NT; ++j) {
+    for (int j = 0; j < NB; ++j) {
       const int n = n0 + j * 16 + r16;
-      if (n < N) out[d * N + n] = from_f32<TO>(expert_act(acc[j][i], g.act) * g.out_scale);
+      if (n >= N) continue;
+      if constexpr (GATED)
+        out[d * N + n] = from_f32<TO>(expert_unit(g, acc[2 * j][i], acc[2 * j + 1][i], w));
+      else
+        out[d * N + n] = from_f32<TO>(expert_act(acc[j][i], g.act) * g.out_scale * w);
     }
   }
 }
@@ -197,7 +228,8 @@ grouped_gemm_bf16_kernel(GroupedArgs g) {
 #define GG_MIN_WAVES 2    // waves a SIMD the register budget is cut for
 #endif
 
-template <typename TO>
+// GATED: a tile is 64 outputs; its 128 weight rows are gate and up rows in turn, 16 each.
+template <typename TO, bool GATED>
 __global__ void __launch_bounds__(256, GG_MIN_WAVES)
 grouped_gemm_bf16_tiled_kernel(GroupedArgs g) {
   __shared__ __attribute__((aligned(16))) bf16_t As[GG_BM * GG_LD];
@@ -206,10 +238,10 @@ grouped_gemm_bf16_tiled_kernel(GroupedArgs g) {
   if (!find_tile<GG_BM>(g.counts, g.E, blockIdx.x, &e, &tile, &count)) return;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int wm = wave >> 1, wn = wave & 1;
-  const int n0 = blockIdx.y * GG_BN;
+  const int n0 = blockIdx.y * (GATED ? GG_BN / 2 : GG_BN);
   const int* mine = g.lists + (size_t)e * g.A;
   const int K = g.K, N = g.N;
-  const bf16_t* wbase = (const bf16_t*)g.W + (size_t)e * N * K;
+  const bf16_t* wbase = (const bf16_t*)g.W + (size_t)e * (GATED ? 2 * N : N) * K;
 
   f32x4_t acc[4][4];
 #pragma unroll
@@ -224,11 +256,12 @@ grouped_gemm_bf16_tiled_kernel(GroupedArgs g) {
   bool a_ok[4], w_ok[4];
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
-    const int r = tile * GG_BM + lrow + 32 * i, n = n0 + lrow + 32 * i;
+    const int r = tile * GG_BM + lrow + 32 * i, tr = lrow + 32 * i;
+    const int n = n0 + (GATED ? (tr >> 5) * 16 + (tr & 15) : tr);
     a_ok[i] = r < count;
     w_ok[i] = n < N;
     arow[i] = (const bf16_t*)g.src + (size_t)(a_ok[i] ? mine[r] / g.src_div : 0) * K;
-    wrow[i] = wbase + (size_t)(w_ok[i] ? n : 0) * K;
+    wrow[i] = wbase + (size_t)(w_ok[i] ? n + (GATED && (tr & 16) ? N : 0) : 0) * K;
   }
   bf16x8_t ra[4], rw[4];
   const bf16x8_t zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
@@ -283,16 +316,26 @@ grouped_gemm_bf16_tiled_kernel(GroupedArgs g) {
       const int row = tile * GG_BM + wm * 64 + i * 16 + (lane >> 4) * 4 + r;
       if (row >= count) continue;
       const size_t d = dst_row(g, mine[row]);
+      const float w = g.row_weight ? g.row_weight[mine[row]] : 1.0f;
+      if constexpr (GATED) {
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int n = n0 + wn * 64 + j * 16 + r16;
-        if (n < N) out[d * N + n] = from_f32<TO>(expert_act(acc[i][j][r], g.act) * g.out_scale);
+        for (int j = 0; j < 4; j += 2) {
+          const int n = n0 + wn * 32 + (j / 2) * 16 + r16;
+          if (n < N) out[d * N + n] = from_f32<TO>(expert_unit(g, acc[i][j][r], acc[i][j + 1][r], w));
+        }
+      } else {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const int n = n0 + wn * 64 + j * 16 + r16;
+          if (n < N) out[d * N + n] = from_f32<TO>(expert_act(acc[i][j][r], g.act) * g.out_scale * w);
+        }
       }
     }
 }
 
-// 32-bit weights (src of either type): 64 x 64 tiles through LDS, plain FMA.
-template <typename TA, typename TO>
+// 32-bit weights (src of either type): 64 x 64 tiles through LDS, plain FMA.  GATED: a tile is 32
+// outputs, a thread's four weight rows are two gate rows and the two up rows that go with them.
+template <typename TA, typename TO, bool GATED>
 __global__ void __launch_bounds__(256)
 grouped_gemm_f32_kernel(GroupedArgs g) {
   __shared__ float As[16][64 + 4];
@@ -300,16 +343,17 @@ grouped_gemm_f32_kernel(GroupedArgs g) {
   int e, tile, count;
   if (!find_tile<64>(g.counts, g.E, blockIdx.x, &e, &tile, &count)) return;
   const int tid = threadIdx.x, tx = tid % 16, ty = tid / 16;
-  const int n0 = blockIdx.y * 64;
+  const int n0 = blockIdx.y * (GATED ? 32 : 64);
   const int* mine = g.lists + (size_t)e * g.A;
   const int K = g.K, N = g.N;
-  const float* W = (const float*)g.W + (size_t)e * N * K;
+  const float* W = (const float*)g.W + (size_t)e * (GATED ? 2 * N : N) * K;
   const int lrow = tid / 4, lk = (tid % 4) * 4;
   const int arow_idx = tile * 64 + lrow;
   const bool a_ok = arow_idx < count;
   const TA* arow = (const TA*)g.src + (size_t)(a_ok ? mine[arow_idx] / g.src_div : 0) * K;
-  const bool w_ok = n0 + lrow < N;
-  const float* wrow = W + (size_t)(w_ok ? n0 + lrow : 0) * K;
+  const int wn = n0 + (GATED ? (lrow / 4) * 2 + (lrow & 1) : lrow);
+  const bool w_ok = wn < N;
+  const float* wrow = W + (size_t)(w_ok ? wn + (GATED && (lrow & 2) ? N : 0) : 0) * K;
   float acc[4][4];
 #pragma unroll
   for (int i = 0; i < 4; ++i)
@@ -343,66 +387,85 @@ grouped_gemm_f32_kernel(GroupedArgs g) {
     const int r = tile * 64 + ty * 4 + i;
     if (r >= count) continue;
     const size_t d = dst_row(g, mine[r]);
+    const float w = g.row_weight ? g.row_weight[mine[r]] : 1.0f;
+    if constexpr (GATED) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int n = n0 + tx * 4 + j;
-      if (n < N) out[d * N + n] = from_f32<TO>(expert_act(acc[i][j], g.act) * g.out_scale);
+      for (int j = 0; j < 2; ++j) {
+        const int n = n0 + tx * 2 + j;
+        if (n < N) out[d * N + n] = from_f32<TO>(expert_unit(g, acc[i][j], acc[i][j + 2], w));
+      }
+    } else {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int n = n0 + tx * 4 + j;
+        if (n < N) out[d * N + n] = from_f32<TO>(expert_act(acc[i][j], g.act) * g.out_scale * w);
+      }
     }
   }
 }
 
 // dtype codes: 0 = float32, 1 = bfloat16.  `src` has `src_rows` rows of K elements; the
 // lists name assignments below n_tokens * top, so src_rows >= n_tokens (src_div == top) or
-// >= n_tokens * top (src_div == 1).
+// >= n_tokens * top (src_div == 1).  With `gate` (see GroupedArgs) W is [experts][2N][K].
 extern "C" int za_grouped_gemm(const void* src, int src_dtype, long long src_rows, const void* W,
                                int w_dtype, const int* lists, const int* counts, void* out,
                                int out_dtype, int n_tokens, int top, int experts, int N, int K,
                                int src_div, int stacked, int act, float out_scale,
-                               hipStream_t stream) {
+                               const float* row_weight, int gate, float bound, float slope,
+                               float offset, hipStream_t stream) {
   if (n_tokens == 0) return 0;
   if (n_tokens < 0 || top <= 0 || experts <= 0 || N <= 0 || K <= 0 || !src || !W || !lists ||
-      !counts || !out || (src_div != 1 && src_div != top) || act < 0 || act > 1)
+      !counts || !out || (src_div != 1 && src_div != top) || act < 0 || act > 1 ||
+      gate < 0 || gate > 3 || (gate && (act || out_scale != 1.0f)))
     return ZA_ERR_ARG;
   const long long A = (long long)n_tokens * top;
   if (src_rows < (src_div == 1 ? A : (long long)n_tokens) || A > 0x7fffffff) return ZA_ERR_ARG;
   if (experts > EX_MAX_EXPERTS) return ZA_ERR_UNSUPPORTED;
   if (stacked && out_dtype != 0) return ZA_ERR_UNSUPPORTED;
   GroupedArgs g{src, W, lists, counts, out, (int)A, n_tokens, top, experts, N, K,
-                src_div, stacked, act, out_scale};
-  const unsigned ntiles = (unsigned)((N + 63) / 64);
+                src_div, stacked, act, out_scale, row_weight, gate, bound, slope, offset};
   if (w_dtype == 1) {
     if (src_dtype != 1 || K % 8 != 0) return ZA_ERR_UNSUPPORTED;
     if (A >= 128LL * experts) {
       // many rows an expert: tiles of 128 x 128 through LDS
-      dim3 grid((unsigned)((A + GG_BM - 1) / GG_BM + experts), (unsigned)((N + GG_BN - 1) / GG_BN));
-      if (out_dtype == 0)
-        hipLaunchKernelGGL((grouped_gemm_bf16_tiled_kernel<float>), grid, dim3(256), 0, stream, g);
-      else if (out_dtype == 1)
-        hipLaunchKernelGGL((grouped_gemm_bf16_tiled_kernel<bf16_t>), grid, dim3(256), 0, stream, g);
-      else
-        return ZA_ERR_UNSUPPORTED;
+      const int columns = gate ? GG_BN / 2 : GG_BN;
+      dim3 grid((unsigned)((A + GG_BM - 1) / GG_BM + experts), (unsigned)((N + columns - 1) / columns));
+#define ZA_GT(TO, GATED) \
+  hipLaunchKernelGGL((grouped_gemm_bf16_tiled_kernel<TO, GATED>), grid, dim3(256), 0, stream, g)
+      if (out_dtype == 0) { if (gate) ZA_GT(float, true); else ZA_GT(float, false); }
+      else if (out_dtype == 1) { if (gate) ZA_GT(bf16_t, true); else ZA_GT(bf16_t, false); }
+      else return ZA_ERR_UNSUPPORTED;
+#undef ZA_GT
       return za_launch_status();
     }
     // a decode batch (an expert has a token or two): tiles of 16 rows
     const bool small = A <= 4LL * experts || A <= 64;
     const int TM = small ? 16 : 64;
-    dim3 grid((unsigned)((A + TM - 1) / TM + experts), ntiles), block(256);
-#define ZA_GG(TMM, TO) \
-  hipLaunchKernelGGL((grouped_gemm_bf16_kernel<TMM, TO>), grid, block, 0, stream, g)
-    if (out_dtype == 0) { if (small) ZA_GG(16, float); else ZA_GG(64, float); }
-    else if (out_dtype == 1) { if (small) ZA_GG(16, bf16_t); else ZA_GG(64, bf16_t); }
+    const int columns = gate && !small ? 32 : 64;
+    dim3 grid((unsigned)((A + TM - 1) / TM + experts), (unsigned)((N + columns - 1) / columns)), block(256);
+#define ZA_GG(TMM, TO)                                                                          \
+  {                                                                                             \
+    if (gate) hipLaunchKernelGGL((grouped_gemm_bf16_kernel<TMM, TO, true>), grid, block, 0, stream, g); \
+    else hipLaunchKernelGGL((grouped_gemm_bf16_kernel<TMM, TO, false>), grid, block, 0, stream, g);     \
+  }
+    if (out_dtype == 0) { if (small) ZA_GG(16, float) else ZA_GG(64, float) }
+    else if (out_dtype == 1) { if (small) ZA_GG(16, bf16_t) else ZA_GG(64, bf16_t) }
     else return ZA_ERR_UNSUPPORTED;
 #undef ZA_GG
     return za_launch_status();
   }
   if (w_dtype != 0) return ZA_ERR_UNSUPPORTED;
-  dim3 grid((unsigned)((A + 63) / 64 + experts), ntiles), block(256);
-#define ZA_GF(TA, TO) \
-  hipLaunchKernelGGL((grouped_gemm_f32_kernel<TA, TO>), grid, block, 0, stream, g)
-  if (src_dtype == 0 && out_dtype == 0) ZA_GF(float, float);
-  else if (src_dtype == 1 && out_dtype == 0) ZA_GF(bf16_t, float);
-  else if (src_dtype == 1 && out_dtype == 1) ZA_GF(bf16_t, bf16_t);
-  else if (src_dtype == 0 && out_dtype == 1) ZA_GF(float, bf16_t);
+  const int columns = gate ? 32 : 64;
+  dim3 grid((unsigned)((A + 63) / 64 + experts), (unsigned)((N + columns - 1) / columns)), block(256);
+#define ZA_GF(TA, TO)                                                                             \
+  {                                                                                               \
+    if (gate) hipLaunchKernelGGL((grouped_gemm_f32_kernel<TA, TO, true>), grid, block, 0, stream, g); \
+    else hipLaunchKernelGGL((grouped_gemm_f32_kernel<TA, TO, false>), grid, block, 0, stream, g);     \
+  }
+  if (src_dtype == 0 && out_dtype == 0) ZA_GF(float, float)
+  else if (src_dtype == 1 && out_dtype == 0) ZA_GF(bf16_t, float)
+  else if (src_dtype == 1 && out_dtype == 1) ZA_GF(bf16_t, bf16_t)
+  else if (src_dtype == 0 && out_dtype == 1) ZA_GF(float, bf16_t)
   else return ZA_ERR_UNSUPPORTED;
 #undef ZA_GF
   return za_launch_status();

@@ -580,3 +580,70 @@ extern "C" int za_embed_pairs(const int* tokens, const void* table, const void* 
 #undef ZA_EMBED_PAIRS
   return za_launch_status();
 }
+
+// The rows that open the stream, normed:  h = table[tokens[t]],
+//   out[t] = h / sqrt(mean(h^2) + eps) * weight
+// in 32-bit, and with `copy` also stored rounded.  One workgroup a token; the row is read a
+// second time from the cache where it does not fit the registers.
+template <typename T, typename TC>
+__global__ void __launch_bounds__(256)
+embed_norm_kernel(const int* __restrict__ tokens, const T* __restrict__ table,
+                  const float* __restrict__ weight, float* __restrict__ out, TC* __restrict__ copy,
+                  int width, int vocab, float eps) {
+  constexpr int KEEP = 8;
+  __shared__ float scratch[16];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  const int tok = tokens[t];
+  // (never read outside the table; an id the host failed to reject poisons its row)
+  const bool ok = tok >= 0 && tok < vocab;
+  const T* row = table + (size_t)(ok ? tok : 0) * width;
+  float* o = out + (size_t)t * width;
+  TC* c = copy ? copy + (size_t)t * width : nullptr;
+  float kept[KEEP];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < KEEP; ++k) {
+    const int i = tid + k * 256;
+    kept[k] = i < width ? to_f32<T>(row[i]) : 0.f;
+    ss += kept[k] * kept[k];
+  }
+  for (int i = tid + KEEP * 256; i < width; i += 256) {
+    const float v = to_f32<T>(row[i]);
+    ss += v * v;
+  }
+  ss = block_sum(ss, scratch);
+  const float f = ok ? 1.0f / sqrtf(ss / (float)width + eps) : __builtin_nanf("");
+#pragma unroll
+  for (int k = 0; k < KEEP; ++k) {
+    const int i = tid + k * 256;
+    if (i < width) {
+      const float h = kept[k] * f * weight[i];
+      o[i] = h;
+      if (c) c[i] = from_f32<TC>(h);
+    }
+  }
+  for (int i = tid + KEEP * 256; i < width; i += 256) {
+    const float h = to_f32<T>(row[i]) * f * weight[i];
+    o[i] = h;
+    if (c) c[i] = from_f32<TC>(h);
+  }
+}
+
+extern "C" int za_embed_norm(const int* tokens, const void* table, int table_dtype,
+                             const float* weight, float* out, void* copy, int copy_dtype,
+                             int n_tokens, int width, int vocab, float eps, hipStream_t stream) {
+  if (n_tokens == 0) return 0;
+  if (n_tokens < 0 || width <= 0 || vocab <= 0 || !tokens || !table || !weight || !out)
+    return ZA_ERR_ARG;
+  dim3 grid(n_tokens), block(256);
+#define ZA_EMBED_NORM(T, TC)                                                                 \
+  hipLaunchKernelGGL((embed_norm_kernel<T, TC>), grid, block, 0, stream, tokens,             \
+                     (const T*)table, weight, out, (TC*)copy, width, vocab, eps)
+  if (table_dtype == 0 && copy_dtype == 0) ZA_EMBED_NORM(float, float);
+  else if (table_dtype == 0 && copy_dtype == 1) ZA_EMBED_NORM(float, bf16_t);
+  else if (table_dtype == 1 && copy_dtype == 0) ZA_EMBED_NORM(bf16_t, float);
+  else if (table_dtype == 1 && copy_dtype == 1) ZA_EMBED_NORM(bf16_t, bf16_t);
+  else return ZA_ERR_UNSUPPORTED;
+#undef ZA_EMBED_NORM
+  return za_launch_status();
+}

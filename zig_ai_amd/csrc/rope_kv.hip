@@ -355,14 +355,14 @@ extern "C" int za_qk_norm_rope_kv_write_wide(const void* qkv, const int* positio
 // kernels above, `dv`, `row_stride` and `magnitude` as there.  nkv == 0: the rows hold queries
 // only, nothing is stored (a layer that reads another layer's keys and values).
 //
-// A workgroup a token.  The row's heads are staged in LDS as floats, pieces of eight elements a
-// thread; the two sums of squares meet once, every thread then norms its own pieces, and the
-// rotation reads a piece and its partners from LDS.  In steps of many tokens the values are
+// A workgroup a token, NP pieces of eight elements a thread, held in registers.  The two sums
+// of squares meet once; every thread norms its own pieces and leaves them in LDS, where the
+// rotation finds a piece's partners.  In steps of many tokens the values are
 // stored by workgroups of their own, first in the grid: a wave takes eight consecutive tokens
 // and, where these lie side by side in one page, stores a head-dim element's eight values with
 // one access.
-template <typename T>
-__global__ void __launch_bounds__(256)
+template <typename T, int NP>
+__global__ void __launch_bounds__(512)
 qk_row_norm_rope_kv_write_kernel(const T* __restrict__ qkv, const int* __restrict__ positions,
                                  const int* __restrict__ slots, const float* __restrict__ q_norm_w,
                                  const float* __restrict__ k_norm_w,
@@ -372,12 +372,13 @@ qk_row_norm_rope_kv_write_kernel(const T* __restrict__ qkv, const int* __restric
                                  float k_count, float magnitude, int page_size, int write_kv,
                                  int n_tokens, int value_blocks) {
   extern __shared__ __attribute__((aligned(16))) float rows_lds[];   // [(nh + nkv) * d][rot]
-  __shared__ float sums[2][4];
+  __shared__ float sums[2][16];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int n_threads = blockDim.x, n_waves = n_threads >> 6;
   const size_t page_elems = (size_t)nkv * page_size * (d + dv);
   const size_t value_base = (size_t)nkv * page_size * d;
   if ((int)blockIdx.x < value_blocks) {
-    const int t0 = ((int)blockIdx.x * 4 + wave) * 8;   // a wave's 8 tokens
+    const int t0 = ((int)blockIdx.x * n_waves + wave) * 8;   // a wave's 8 tokens
     if (t0 >= n_tokens) return;
     int slot[8];
 #pragma unroll
@@ -385,32 +386,38 @@ qk_row_norm_rope_kv_write_kernel(const T* __restrict__ qkv, const int* __restric
     bool side_by_side = page_size % 8 == 0 && slot[0] >= 0 && slot[0] % 8 == 0;
 #pragma unroll
     for (int j = 1; j < 8; ++j) side_by_side = side_by_side && slot[j] == slot[0] + j;
-    const int pieces = nkv * dv / 8;
+    constexpr int E = 16 / (int)sizeof(T);             // elements of a 16-byte piece
+    typedef T piece_t __attribute__((ext_vector_type(E)));
+    typedef T run_t __attribute__((ext_vector_type(8)));
+    const int pieces = nkv * dv / E;
+    const T* src = qkv + (size_t)t0 * row_stride + (size_t)(nh + nkv) * d;
     for (int piece = lane; piece < pieces; piece += 64) {
-      float x[8][8];
+      piece_t x[8];
 #pragma unroll
-      for (int j = 0; j < 8; ++j)
-        if (t0 + j < n_tokens)
-          load8<T>(qkv + (size_t)(t0 + j) * row_stride + (size_t)(nh + nkv) * d + piece * 8, x[j]);
+      for (int j = 0; j < 8; ++j)      // (a token beyond the last reads the last one again)
+        x[j] = *reinterpret_cast<const piece_t*>(
+            src + (size_t)(min(t0 + j, n_tokens - 1) - t0) * row_stride + piece * E);
       if (side_by_side) {
         T* dst = kv_cache + (size_t)(slot[0] / page_size) * page_elems + value_base +
-                 (size_t)piece * 8 * page_size + slot[0] % page_size;
+                 (size_t)piece * E * page_size + slot[0] % page_size;
 #pragma unroll
-        for (int i = 0; i < 8; ++i) {
-          float run[8];
+        for (int i = 0; i < E; ++i) {
+          run_t run;
 #pragma unroll
           for (int j = 0; j < 8; ++j) run[j] = x[j][i];
-          store8<T>(dst + (size_t)i * page_size, run);
+          *reinterpret_cast<run_t*>(dst + (size_t)i * page_size) = run;
         }
       } else {
+#pragma unroll 1
+        for (int j = 0; j < 8 && t0 + j < n_tokens; ++j) {   // (a rare group: tokens one by one)
+          const int place = slots[t0 + j];
+          if (place < 0) continue;
+          const piece_t one = *reinterpret_cast<const piece_t*>(src + (size_t)j * row_stride + piece * E);
+          T* dst = kv_cache + (size_t)(place / page_size) * page_elems + value_base +
+                   (size_t)piece * E * page_size + place % page_size;
 #pragma unroll
-        for (int j = 0; j < 8; ++j)
-          if (slot[j] >= 0) {
-            T* dst = kv_cache + (size_t)(slot[j] / page_size) * page_elems + value_base +
-                     (size_t)piece * 8 * page_size + slot[j] % page_size;
-#pragma unroll
-            for (int i = 0; i < 8; ++i) dst[(size_t)i * page_size] = from_f32<T>(x[j][i]);
-          }
+          for (int i = 0; i < E; ++i) dst[(size_t)i * page_size] = one[i];
+        }
       }
     }
     return;
@@ -423,19 +430,30 @@ qk_row_norm_rope_kv_write_kernel(const T* __restrict__ qkv, const int* __restric
   float* cs_tab = rows_lds + (size_t)(nh + nkv) * d;
   float* sn_tab = cs_tab + half;
 
-  float qs = 0.f, ks = 0.f;
-  for (int piece = tid; piece < pieces; piece += 256) {
-    float x[8];
-    load8<T>(row + piece * 8, x);
-    const float ss = rope_sum_squares8(x);
-    if (piece < q_pieces) qs += ss; else ks += ss;
-    store8<float>(rows_lds + piece * 8, x);
+  // everything the token needs is requested at once
+  const int slot = write_kv ? slots[t] : -1;
+  float x[NP][8], w[NP][8];
+#pragma unroll
+  for (int j = 0; j < NP; ++j) {
+    const int piece = tid + j * n_threads;
+    if (piece < pieces) {
+      load8<T>(row + piece * 8, x[j]);
+      load8<float>(piece < q_pieces ? q_norm_w + piece * 8 : k_norm_w + (piece - q_pieces) * 8, w[j]);
+    }
   }
-  for (int p = tid; p < half; p += 256) {
+  for (int p = tid; p < half; p += n_threads) {
     float cs, sn;
     rope_angle(positions[t], inv_freq[p], &cs, &sn);
     cs_tab[p] = cs * magnitude;
     sn_tab[p] = sn * magnitude;
+  }
+  float qs = 0.f, ks = 0.f;
+#pragma unroll
+  for (int j = 0; j < NP; ++j) {
+    const int piece = tid + j * n_threads;
+    if (piece >= pieces) continue;
+    const float ss = rope_sum_squares8(x[j]);
+    if (piece < q_pieces) qs += ss; else ks += ss;
   }
   qs = wave_sum(qs);
   ks = wave_sum(ks);
@@ -444,50 +462,67 @@ qk_row_norm_rope_kv_write_kernel(const T* __restrict__ qkv, const int* __restric
     sums[1][wave] = ks;
   }
   __syncthreads();
-  const float q_scale =
-      1.0f / sqrtf((sums[0][0] + sums[0][1] + sums[0][2] + sums[0][3]) / q_count + eps);
-  const float k_scale =
-      1.0f / sqrtf((sums[1][0] + sums[1][1] + sums[1][2] + sums[1][3]) / k_count + eps);
-  for (int piece = tid; piece < pieces; piece += 256) {
-    const bool is_q = piece < q_pieces;
-    float x[8], w[8];
-    load8<float>(rows_lds + piece * 8, x);
-    load8<float>(is_q ? q_norm_w + piece * 8 : k_norm_w + (piece - q_pieces) * 8, w);
-    rope_scale8(x, is_q ? q_scale : k_scale, w);
-    store8<float>(rows_lds + piece * 8, x);
+  qs = ks = 0.f;
+  for (int i = 0; i < n_waves; ++i) {
+    qs += sums[0][i];
+    ks += sums[1][i];
+  }
+  const float q_scale = 1.0f / sqrtf(qs / q_count + eps);
+  const float k_scale = 1.0f / sqrtf(ks / k_count + eps);
+#pragma unroll
+  for (int j = 0; j < NP; ++j) {
+    const int piece = tid + j * n_threads;
+    if (piece >= pieces) continue;
+    rope_scale8(x[j], piece < q_pieces ? q_scale : k_scale, w[j]);
+    store8<float>(rows_lds + piece * 8, x[j]);
   }
   __syncthreads();
-  const int slot = write_kv ? slots[t] : -1;
   T* pg = slot >= 0 ? kv_cache + (size_t)(slot / page_size) * page_elems : nullptr;
   const int off = slot >= 0 ? slot % page_size : 0;
-  for (int piece = tid; piece < pieces; piece += 256) {
+  const bool whole_pieces = !adjacent && half % 8 == 0;   // a piece's partners are one piece
+#pragma unroll
+  for (int j = 0; j < NP; ++j) {
+    const int piece = tid + j * n_threads;
+    if (piece >= pieces) continue;
     const int head = piece * 8 / d, e0 = piece * 8 % d;
     const float* h = rows_lds + (size_t)head * d;
-    float x[8];
-    load8<float>(h + e0, x);
-    if (e0 < rot) {
+    if (e0 < rot && whole_pieces) {
+      const bool low = e0 < half;
+      float other[8], cs[8], sn[8];
+      load8<float>(h + (low ? e0 + half : e0 - half), other);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        cs[i] = cs_tab[(low ? e0 : e0 - half) + i];
+        sn[i] = sn_tab[(low ? e0 : e0 - half) + i];
+      }
+#pragma unroll
+      for (int i = 0; i < 8; ++i)
+        x[j][i] = low ? rope_rotate_low(x[j][i], other[i], cs[i], sn[i])
+                      : rope_rotate_high(x[j][i], other[i], cs[i], sn[i]);
+    } else if (e0 < rot) {
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
         const int e = e0 + i;
         if (e >= rot) continue;
         if (adjacent) {
           const float other = h[e ^ 1], cs = cs_tab[e >> 1], sn = sn_tab[e >> 1];
-          x[i] = (e & 1) ? rope_rotate_high(x[i], other, cs, sn) : rope_rotate_low(x[i], other, cs, sn);
+          x[j][i] = (e & 1) ? rope_rotate_high(x[j][i], other, cs, sn)
+                            : rope_rotate_low(x[j][i], other, cs, sn);
         } else if (e < half) {
-          x[i] = rope_rotate_low(x[i], h[e + half], cs_tab[e], sn_tab[e]);
+          x[j][i] = rope_rotate_low(x[j][i], h[e + half], cs_tab[e], sn_tab[e]);
         } else {
-          x[i] = rope_rotate_high(x[i], h[e - half], cs_tab[e - half], sn_tab[e - half]);
+          x[j][i] = rope_rotate_high(x[j][i], h[e - half], cs_tab[e - half], sn_tab[e - half]);
         }
       }
     }
     if (piece < q_pieces)
-      store8<T>(q_out + (size_t)t * nh * d + piece * 8, x);
+      store8<T>(q_out + (size_t)t * nh * d + piece * 8, x[j]);
     else if (pg)
-      store8<T>(pg + ((size_t)(head - nh) * page_size + off) * d + e0, x);
+      store8<T>(pg + ((size_t)(head - nh) * page_size + off) * d + e0, x[j]);
   }
   if (pg && value_blocks == 0) {
     const T* v = row + (size_t)(nh + nkv) * d;
-    for (int i = tid; i < nkv * dv; i += 256) pg[value_base + (size_t)i * page_size + off] = v[i];
+    for (int i = tid; i < nkv * dv; i += n_threads) pg[value_base + (size_t)i * page_size + off] = v[i];
   }
 }
 
@@ -511,10 +546,17 @@ extern "C" int za_qk_row_norm_rope_kv_write(const void* qkv, const int* position
     return ZA_ERR_ARG;
   const size_t shmem = ((size_t)(nh + nkv) * d + rot) * sizeof(float);
   if (shmem > RK_ROW_MAX_LDS) return ZA_ERR_UNSUPPORTED;
-  const int value_blocks = (write_kv && n_tokens >= RK_VALUE_BLOCKS_FROM) ? (n_tokens + 31) / 32 : 0;
-#define ZA_RK_ROW(T)                                                                             \
+  const int pieces = nh * d / 8 + (write_kv ? nkv * d / 8 : 0);
+  int np = 1;
+  while (np < 8 && pieces > np * 512) np *= 2;
+  if (pieces > np * 1024) return ZA_ERR_UNSUPPORTED;
+  const int threads = ((pieces + np - 1) / np + 63) / 64 * 64;
+  const int per_block = threads / 64 * 8;   // tokens whose values a workgroup stores
+  const int value_blocks =
+      (write_kv && n_tokens >= RK_VALUE_BLOCKS_FROM) ? (n_tokens + per_block - 1) / per_block : 0;
+#define ZA_RK_ROW_NP(T, NP)                                                                      \
   {                                                                                              \
-    auto kernel = qk_row_norm_rope_kv_write_kernel<T>;                                           \
+    auto kernel = qk_row_norm_rope_kv_write_kernel<T, NP>;                                       \
     static size_t allowed = 48 * 1024;                                                           \
     if (shmem > allowed) {                                                                       \
       const hipError_t e = hipFuncSetAttribute(                                                  \
@@ -522,14 +564,22 @@ extern "C" int za_qk_row_norm_rope_kv_write(const void* qkv, const int* position
       if (e != hipSuccess) return (int)e;                                                        \
       allowed = shmem;                                                                           \
     }                                                                                            \
-    hipLaunchKernelGGL(kernel, dim3(n_tokens + value_blocks), dim3(256), shmem, stream,          \
+    hipLaunchKernelGGL(kernel, dim3(n_tokens + value_blocks), dim3(threads), shmem, stream,      \
                        (const T*)qkv, positions, slots, q_norm_w, k_norm_w, inv_freq, (T*)q_out, \
                        (T*)kv_cache, nh, nkv, d, dv, row_stride, rot, adjacent, eps, q_count,    \
                        k_count, magnitude, page_size, write_kv, n_tokens, value_blocks);         \
     return za_launch_status();                                                                   \
   }
+#define ZA_RK_ROW(T)                  \
+  {                                   \
+    if (np == 1) ZA_RK_ROW_NP(T, 1)   \
+    if (np == 2) ZA_RK_ROW_NP(T, 2)   \
+    if (np == 4) ZA_RK_ROW_NP(T, 4)   \
+    ZA_RK_ROW_NP(T, 8)                \
+  }
   if (dtype == 0) ZA_RK_ROW(float)
   if (dtype == 1) ZA_RK_ROW(bf16_t)
 #undef ZA_RK_ROW
+#undef ZA_RK_ROW_NP
   return ZA_ERR_UNSUPPORTED;
 }

@@ -107,6 +107,12 @@ class DecoderModel:
                              for i, part in enumerate(getattr(spec, "stream_parts", ()))]
         for p in self.stream_parts:
             note(p)
+        # (an embedding may leave its rows rounded, too, for a first block that reads them so)
+        self.embedding_rounds = bool(getattr(self.embedding, "leaves_rounded", False))
+        if self.embedding_rounds:
+            first = spec.schedule[0]
+            self.embedding.rounded_wanted = first.before is None and \
+                bool(getattr(self.blocks[first.layer], "leaves_rounded", False))
         self.final_norm = make("norm", spec.final_norm, ("final_norm",))
         self.head = make("head", spec.lm_head, ("lm_head",))
         note(self.final_norm)
@@ -261,7 +267,8 @@ class DecoderModel:
                  taps: Optional[List[Dict[str, torch.Tensor]]]) -> torch.Tensor:
         step.rounded = None
         residual = self.embedding.forward(step.token_ids, step, views[len(self.schedule)]) \
-            if self.embedding_keeps else self.embedding.forward(step.token_ids)
+            if self.embedding_keeps else self.embedding.forward(step.token_ids, step) \
+            if self.embedding_rounds else self.embedding.forward(step.token_ids)
         pending = None
         if taps is not None:
             taps.append({"stream": residual.clone()})

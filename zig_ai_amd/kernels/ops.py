@@ -169,7 +169,8 @@ _SIGNATURES = {
                                      c_void_p, c_void_p],
     ("experts", "za_grouped_gemm"): [c_void_p, c_int, c_longlong, c_void_p, c_int, c_void_p,
                                      c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
-                                     c_int, c_int, c_int, c_float, c_void_p],
+                                     c_int, c_int, c_int, c_float, c_void_p, c_int, c_float,
+                                     c_float, c_float, c_void_p],
     ("activation", "za_softcap"): [c_void_p, c_float, c_longlong, c_void_p],
     ("activation", "za_table_gate"): [c_void_p, c_int, c_void_p, c_void_p, c_int, c_int, c_int,
                                       c_int, c_void_p, c_int, c_int, c_int, c_void_p],
@@ -178,6 +179,8 @@ _SIGNATURES = {
     ("norm", "za_embed_pairs"): [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p,
                                  c_void_p, c_void_p, c_longlong, c_longlong, c_longlong, c_longlong,
                                  c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p],
+    ("norm", "za_embed_norm"): [c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_int,
+                                c_int, c_int, c_float, c_void_p],
     ("recurrent", "za_channel_decay_prepare"): [c_void_p, c_int, c_int, c_int, c_int, c_int, c_int,
                                                 c_int, c_void_p, c_int, c_void_p, c_float, c_float,
                                                 c_void_p, c_int, c_int, c_int, c_int, c_int,
@@ -344,6 +347,26 @@ def embed_gather(tokens: torch.Tensor, table: torch.Tensor) -> torch.Tensor:
                                         tokens.numel(), width, vocab, _stream())
     _check(rc, "embed_gather")
     return out
+
+
+def embed_norm(tokens: torch.Tensor, table: torch.Tensor, weight: torch.Tensor, eps: float,
+               copy_dtype: Optional[torch.dtype] = None):
+    """``h / sqrt(mean(h^2) + eps) * weight`` for the rows ``h = table[tokens]``, as 32-bit rows;
+    with ``copy_dtype`` also rounded to that type.  Returns ``(rows, copy or None)``."""
+    _need(tokens, "tokens", torch.int32)
+    _need(table, "table", (torch.float32, torch.bfloat16))
+    if table.dim() != 2:
+        raise KernelError(f"table must be [vocab, width], got {tuple(table.shape)}")
+    T, (vocab, width) = tokens.numel(), table.shape
+    _need(weight, "weight", torch.float32, (width,))
+    out = torch.empty((T, width), dtype=torch.float32, device=table.device)
+    copy = None if copy_dtype is None else torch.empty((T, width), dtype=copy_dtype,
+                                                       device=table.device)
+    rc = _fn("norm", "za_embed_norm")(
+        _ptr(tokens), _ptr(table), _code(table.dtype), _ptr(weight), _ptr(out), _ptr(copy),
+        _code(copy_dtype or torch.float32), T, width, vocab, float(eps), _stream())
+    _check(rc, "embed_norm")
+    return out, copy
 
 
 def embed_pairs(tokens: torch.Tensor, table: torch.Tensor, pairs: torch.Tensor,
@@ -641,7 +664,8 @@ library_tuning = os.environ.get("ZIG_AI_GEMM_TUNE", "1") != "0"
 
 def _library_matmul(x: torch.Tensor, weight: torch.Tensor, out_dtype: torch.dtype,
                     splits: int, tune: Optional[bool] = None,
-                    added_to: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+                    added_to: Optional[torch.Tensor] = None,
+                    into: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """``x @ weight^T`` through the GEMM library (csrc/blaslt.hip): ``[M, N]``, or the
     stack ``[splits, M, N]`` of 32-bit partial sums over ranges of K, or, with ``added_to``
     (32-bit ``[M, N]``), that tensor with the product added to it.  ``None`` when
@@ -658,7 +682,8 @@ def _library_matmul(x: torch.Tensor, weight: torch.Tensor, out_dtype: torch.dtyp
         out, kind = added_to, 2
     else:
         shape = (splits, M, N) if splits > 1 else (M, N)
-        out = torch.empty(shape, dtype=torch.float32 if f32 else torch.bfloat16, device=x.device)
+        out = into if into is not None else \
+            torch.empty(shape, dtype=torch.float32 if f32 else torch.bfloat16, device=x.device)
         kind = 1 if f32 else 0
     rc = _fn("blaslt", "za_lt_matmul")(_ptr(x), _ptr(weight), _ptr(out), M, N, K, kind,
                                        splits, 1 if (library_tuning if tune is None else tune) else 0,
@@ -749,7 +774,8 @@ def linear(x, weight: torch.Tensor, bias: Optional[torch.Tensor] = None,
            out_dtype: Optional[torch.dtype] = None, force_tiled: bool = False,
            partial_ok: bool = False,
            accumulate: Optional[torch.Tensor] = None,
-           tune: Optional[bool] = None) -> Optional[torch.Tensor]:
+           tune: Optional[bool] = None,
+           into: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """``x [M, K] @ weight[N, K]^T + bias`` with 32-bit accumulation.
 
     bfloat16 weights use the matrix-core kernels of csrc/gemm.hip up to
@@ -770,7 +796,12 @@ def linear(x, weight: torch.Tensor, bias: Optional[torch.Tensor] = None,
     rounding only); otherwise the product comes back as usual and the caller adds it.
 
     ``tune``: whether the GEMM library may time its candidates at this shape's first call
-    (``None``: the process's default, ``library_tuning``)."""
+    (``None``: the process's default, ``library_tuning``).  ``into``: a contiguous ``[M, N]`` of
+    the result's type to write to (a product without bias that neither adds to a stream nor
+    comes back in ranges)."""
+    if into is not None and (partial_ok or accumulate is not None or bias is not None
+                             or isinstance(x, (NormedRows, MergedRows))):
+        raise KernelError("a product into a given tensor is a plain one")
     if len(x.shape) != 2 or weight.dim() != 2:
         raise KernelError(f"linear takes x [M, K] and weight [N, K], got {tuple(x.shape)} and "
                           f"{tuple(weight.shape)}")
@@ -863,8 +894,10 @@ def linear(x, weight: torch.Tensor, bias: Optional[torch.Tensor] = None,
     if bias is not None:
         _need(bias, "bias", torch.float32, (N,))
     out_dtype = out_dtype or x.dtype
+    if into is not None:
+        _need(into, "into", out_dtype, (M, N))
     if weight.dtype == torch.float32:
-        out = torch.empty((M, N), dtype=out_dtype, device=x.device)
+        out = into if into is not None else torch.empty((M, N), dtype=out_dtype, device=x.device)
         rc = _fn("gemm", "za_gemm_f32")(_ptr(x), _code(x.dtype), _ptr(weight), _ptr(bias), _ptr(out),
                                         _code(out_dtype), M, N, K, _stream())
         _check(rc, "gemm_f32", f"M={M} N={N} K={K}")
@@ -905,12 +938,13 @@ def linear(x, weight: torch.Tensor, bias: Optional[torch.Tensor] = None,
         return stack
     if library:
         # (with ranges of K: one batched product, [P, M, K/P] x [P, K/P, N])
-        out = _library_matmul(x, weight, out_dtype, splits, tune)
+        out = _library_matmul(x, weight, out_dtype, splits, tune,
+                              **({"into": into} if into is not None else {}))
         if out is not None:
             _note("linear", M=M, N=N, K=K, norm_in_product=False, added_to_stream=False,
                   partial_sums=splits, out=out.dtype)
             return out
-    out = torch.empty((M, N), dtype=out_dtype, device=x.device)
+    out = into if into is not None else torch.empty((M, N), dtype=out_dtype, device=x.device)
     rc = _fn("gemm", "za_gemm_bf16")(_ptr(x), _ptr(weight), _ptr(bias), _ptr(out),
                                      _code(out_dtype), M, N, K, 1 if force_tiled else 0,
                                      _stream())
@@ -2400,13 +2434,20 @@ EXPERT_ACTIVATIONS = {None: 0, "relu2": 1}
 def grouped_linear(src: torch.Tensor, weights: torch.Tensor, lists: torch.Tensor,
                    counts: torch.Tensor, n_tokens: int, per_token: bool, stacked: bool = False,
                    activation: Optional[str] = None, out_scale: float = 1.0,
-                   out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
+                   out_dtype: Optional[torch.dtype] = None, gate: Optional[str] = None,
+                   bounded: Optional[Tuple[float, float, float]] = None,
+                   row_weight: Optional[torch.Tensor] = None,
+                   out: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Every assignment's row times its expert's weight: ``weights [experts, N, K]``,
     ``src [T, K]`` (``per_token``: assignment ``a`` reads row ``a // top``) or ``[T*top, K]``
     (one row an assignment).  Returns ``[T*top, N]`` in assignment order, or with ``stacked``
     32-bit ``[top, T, N]``: a stack of partial results that ``add_rmsnorm`` /
     ``add_layernorm`` / ``stream_add_`` add up.  ``activation``: None or ``relu2`` (the square
-    of relu), applied before ``out_scale``."""
+    of relu), applied before ``out_scale``.  ``gate`` (one of ``GATE_ACTIVATIONS``) or ``bounded =
+    (limit, alpha, up_offset)``: ``weights [experts, 2N, K]`` are gate rows and up rows, and the
+    result is the gated unit (``gated_unit`` / ``clamped_glu``) of their 32-bit sums, ``N`` columns.
+    ``row_weight`` (32-bit, one an assignment) multiplies the result, or with a gate the sums
+    ahead of it.  ``out``: write there."""
     if activation not in EXPERT_ACTIVATIONS:
         raise KernelError(f"activation must be None or relu2, got {activation!r}")
     _need(weights, "weights", (torch.float32, torch.bfloat16))
@@ -2415,6 +2456,14 @@ def grouped_linear(src: torch.Tensor, weights: torch.Tensor, lists: torch.Tensor
     E, N, K = weights.shape
     _need(lists, "lists", torch.int32)
     _need(counts, "counts", torch.int32, (E,))
+    gate_code, bounds = 0, (0.0, 0.0, 0.0)
+    if gate is not None or bounded is not None:
+        if activation is not None or N % 2 or (gate is not None and gate not in GATE_ACTIVATIONS):
+            raise KernelError(f"a gated product takes gate and up rows and one of "
+                              f"{sorted(GATE_ACTIVATIONS)}, got {gate!r} with {N} rows")
+        N //= 2
+        gate_code = 1 + (BOUNDED_UNIT if bounded is not None else GATE_ACTIVATIONS[gate])
+        bounds = tuple(float(v) for v in bounded) if bounded is not None else bounds
     if lists.dim() != 2 or lists.shape[0] != E or n_tokens <= 0 or lists.shape[1] % n_tokens:
         raise KernelError(f"lists has shape {tuple(lists.shape)} for {E} experts and {n_tokens} tokens")
     top = lists.shape[1] // n_tokens
@@ -2423,11 +2472,19 @@ def grouped_linear(src: torch.Tensor, weights: torch.Tensor, lists: torch.Tensor
         raise KernelError("bfloat16 expert weights need bfloat16 rows and K a multiple of 8")
     out_dtype = torch.float32 if stacked else (out_dtype or src.dtype)
     shape = (top, n_tokens, N) if stacked else (n_tokens * top, N)
-    out = torch.empty(shape, dtype=out_dtype, device=src.device)
+    if row_weight is not None:
+        _need(row_weight, "row_weight", torch.float32)
+        if row_weight.numel() != n_tokens * top:
+            raise KernelError(f"row_weight holds {row_weight.numel()} numbers for {n_tokens * top} rows")
+    if out is None:
+        out = torch.empty(shape, dtype=out_dtype, device=src.device)
+    else:
+        _need(out, "out", out_dtype, shape)
     rc = _fn("experts", "za_grouped_gemm")(
         _ptr(src), _code(src.dtype), src.shape[0], _ptr(weights), _code(weights.dtype), _ptr(lists),
         _ptr(counts), _ptr(out), _code(out_dtype), n_tokens, top, E, N, K, top if per_token else 1,
-        1 if stacked else 0, EXPERT_ACTIVATIONS[activation], float(out_scale), _stream())
+        1 if stacked else 0, EXPERT_ACTIVATIONS[activation], float(out_scale), _ptr(row_weight),
+        gate_code, *bounds, _stream())
     _check(rc, "grouped_linear", f"E={E} N={N} K={K} tokens={n_tokens} top={top}")
     return out
 

@@ -55,7 +55,19 @@ class TokenEmbedding(Part):
             if self.pair_weight.dtype != self.weight.dtype:
                 self.weight, self.pair_weight = self.weight.float(), self.pair_weight.float()
 
+    # whether the first block reads the stream rounded (the model sets it): the kernel that
+    # makes the rows then leaves such a copy in ``step.rounded``
+    leaves_rounded = True
+    rounded_wanted = False
+
     def forward(self, token_ids: torch.Tensor, step=None, cache=None) -> torch.Tensor:
+        if self.norm_weight is not None and self.pair is None:
+            rounded = self.rounded_wanted and step is not None and self.runtime.dtype != torch.float32
+            x, copy = ops.embed_norm(token_ids, self.weight, self.norm_weight, self.norm_eps,
+                                     self.runtime.dtype if rounded else None)
+            if rounded:
+                step.rounded = copy
+            return x
         if self.pair is not None:
             rounded = self.runtime.dtype if self.runtime.dtype != torch.float32 \
                 and self.norm_weight is None else None

@@ -101,9 +101,12 @@ class RoutedExperts(FeedForward):
     one more expert of that width runs for every token, times ``sigmoid(Wsg x)`` (one number
     a token) when ``shared_gate``.  The router's product and everything after it up to the
     weights is 32-bit; the weighted sum is taken in 32-bit in a fixed order.  A
-    weight on the input is applied to the gate|up product (the same numbers: there are no
-    biases) in front of the bounds; the experts' results then add up without weights, as a
-    stack of partial sums where the arrangement takes one (``partial_ok``).
+    weight on the input is applied to the gate|up product's sums (the same numbers: there are no
+    biases) in front of the bounds.  Where the arrangement takes a stack of partial sums
+    (``partial_ok``) and there are neither identity outputs nor a gate on the shared expert, the
+    experts' first product applies the gate to its own sums, the second one writes its results
+    already weighted, one plane a choice, and the shared expert's result is one plane more: the
+    kernel that norms the sum adds them up.
 
     Nothing is looked at on the host: the router's choice becomes per-expert lists on the
     device and two grouped products run every expert's rows in one launch each."""
@@ -203,32 +206,46 @@ class RoutedExperts(FeedForward):
         if self.experts:
             # an output beyond the experts that have weights is in nobody's list
             lists, counts = ops.expert_lists(None, chosen, T, self.experts)
+            on_input = self.weight_on == "input"
+            bounded = (self.bound, self.slope, self.offset) if self.activation == "bounded_glu" else None
+            if self.partial_ok and not self.identity and not self.shared_gated:
+                a = ops.grouped_linear(x, self.gate_up, lists, counts, T, per_token=True,
+                                       out_dtype=x.dtype, bounded=bounded,
+                                       gate=None if bounded else self.activation,
+                                       row_weight=weight if on_input else None)
+                planes = self.top + (self.shared_gate_up is not None)
+                out = torch.empty((planes, T, self.down.shape[1]), dtype=torch.float32, device=x.device)
+                ops.grouped_linear(a, self.down, lists, counts, T, per_token=False, stacked=True,
+                                   out=out[:self.top], row_weight=None if on_input else weight)
+                if self.shared_gate_up is not None:
+                    self._shared(x, into=out[self.top])
+                return out
+            # (where the rows are combined by a kernel of its own the gate has one, too: the
+            # product's columns are rounded to the run's type in between)
             a = ops.grouped_linear(x, self.gate_up, lists, counts, T, per_token=True,
                                    out_dtype=x.dtype)
-            if self.activation == "bounded_glu":
-                a = ops.clamped_glu(a, self.bound, self.slope, self.offset,
-                                    weight if self.weight_on == "input" else None)
+            if bounded:
+                a = ops.clamped_glu(a, *bounded, weight if on_input else None)
             else:
                 a = ops.gated_unit(a, self.activation)
-            # (nothing but the experts' own results to add up: left to the next kernel)
-            stacked = self.partial_ok and self.weight_on == "input" and not self.identity \
-                and self.shared_gate_up is None
             out = ops.grouped_linear(a, self.down, lists, counts, T, per_token=False,
-                                     stacked=stacked, out_dtype=torch.float32)
-            if stacked:
-                return out
-        shared = None
-        if self.shared_gate_up is not None:
-            if x.dtype == torch.bfloat16 and self.shared_gate_up.dtype == torch.bfloat16 \
-                    and T <= 16 and x.shape[1] <= 8192:
-                # a decode batch: the gate is applied to the projection's accumulators
-                s = ops.linear_swiglu(x, self.shared_gate_up, self.activation)
-            else:
-                s = ops.gated_unit(ops.linear(x, self.shared_gate_up, tune=tune), self.activation)
-            shared = ops.linear(s, self.shared_down, out_dtype=torch.float32, tune=tune)
+                                     out_dtype=torch.float32)
+        shared = self._shared(x) if self.shared_gate_up is not None else None
         return ops.experts_combine(out, chosen, weight, x, self.experts, shared,
                                    logits if self.shared_gated else None, self.outputs,
                                    weigh=self.weight_on == "output")
+
+    def _shared(self, x, into=None):
+        """The shared expert's result, 32-bit."""
+        if x.dtype == torch.bfloat16 and self.shared_gate_up.dtype == torch.bfloat16 \
+                and x.shape[0] <= 16 and x.shape[1] <= 8192:
+            # a decode batch: the gate is applied to the projection's accumulators
+            s = ops.linear_swiglu(x, self.shared_gate_up, self.activation)
+        else:
+            s = ops.gated_unit(ops.linear(x, self.shared_gate_up, tune=self.runtime.tune),
+                               self.activation)
+        return ops.linear(s, self.shared_down, out_dtype=torch.float32, tune=self.runtime.tune,
+                          into=into)
 
 
 register_feed_forward(RoutedExperts.kind, RoutedExperts)

@@ -104,8 +104,9 @@ class ClampedGLU(FeedForward):
         y = (g * sigmoid(alpha * g) * (u + up_offset)) Wd^T
 
     ``limit`` (none if 0), ``alpha`` and ``up_offset`` come from ``params``.  Gate and up
-    weights are one matrix, as in ``SwiGLU``.  In a decode batch the product applies the unit to
-    its own sums, otherwise the unit is a kernel of its own."""
+    weights are one matrix, as in ``SwiGLU``; the unit is a kernel of its own, or with
+    ``unit_in_product`` applied by a decode batch's product to its own 32-bit sums (which the
+    kernel of its own reads rounded to the run's type)."""
 
     kind = "clamped_glu"
     graph_safe = True
@@ -122,12 +123,13 @@ class ClampedGLU(FeedForward):
         self.limit = float(params.get("limit") or 0.0)
         self.alpha = float(params.get("alpha", 1.0))
         self.up_offset = float(params.get("up_offset", 0.0))
+        self.unit_in_product = bool(params.get("unit_in_product", False))
         self.gate_up = ops.projection_weight(fuse_rows(tensors["gate.weight"], tensors["up.weight"]))
         self.down = ops.projection_weight(tensors["down.weight"])
 
     def forward(self, x, step=None):
-        if x.dtype == torch.bfloat16 and self.gate_up.dtype == torch.bfloat16 \
-                and x.shape[0] <= 16 and x.shape[1] <= 8192:
+        if self.unit_in_product and x.dtype == torch.bfloat16 \
+                and self.gate_up.dtype == torch.bfloat16 and x.shape[0] <= 16 and x.shape[1] <= 8192:
             a = ops.linear_swiglu(x, self.gate_up, bounded=(self.limit, self.alpha, self.up_offset))
         else:
             a = ops.clamped_glu(ops.linear(x, self.gate_up, tune=self.runtime.tune), self.limit,
