@@ -149,15 +149,19 @@ __global__ void __launch_bounds__(256)
 grouped_gemm_bf16_kernel(GroupedArgs g) {
   constexpr int WM = TM / 16;          // waves along the rows
   constexpr int WN = 4 / WM;           // waves along the columns
-  // 16-column blocks of the output a wave, and its tiles of weight rows (gate and up in turn)
-  constexpr int NB = GATED ? (TM == 16 ? 1 : 2) : 4 / WN;
-  constexpr int NT = GATED ? 2 * NB : NB;
+  // 16-column blocks of the output a wave, and its tiles of weight rows: with a gate a block has
+  // two, gate and up rows; in a decode batch (PAIRED) they are two neighbouring waves' and meet
+  // in LDS, so that as many waves stream weights as without a gate
+  constexpr bool PAIRED = GATED && TM == 16;
+  constexpr int NB = GATED ? (PAIRED ? 1 : 2) : 4 / WN;
+  constexpr int NT = GATED && !PAIRED ? 2 * NB : NB;
+  [[maybe_unused]] __shared__ float up_sums[PAIRED ? 2 : 1][64][4];
   int e, tile, count;
   if (!find_tile<TM>(g.counts, g.E, blockIdx.x, &e, &tile, &count)) return;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int wm = wave % WM, wn = wave / WM;
   const int r16 = lane & 15, kq = lane >> 4;
-  const int n0 = blockIdx.y * (WN * NB * 16) + wn * NB * 16;
+  const int n0 = PAIRED ? blockIdx.y * 32 + (wn >> 1) * 16 : blockIdx.y * (WN * NB * 16) + wn * NB * 16;
   const int* mine = g.lists + (size_t)e * g.A;
   const int K = g.K, N = g.N;
 
@@ -170,8 +174,9 @@ grouped_gemm_bf16_kernel(GroupedArgs g) {
 #pragma unroll
   for (int j = 0; j < NT; ++j) {
     const int n = n0 + (GATED ? j / 2 : j) * 16 + r16;
+    const bool up = GATED && ((PAIRED ? wn : j) & 1);
     col_ok[j] = n < N;
-    wrow[j] = wbase + (size_t)(col_ok[j] ? n + (GATED && (j & 1) ? N : 0) : 0) * K;
+    wrow[j] = wbase + (size_t)(col_ok[j] ? n + (up ? N : 0) : 0) * K;
   }
   f32x4_t acc[NT];
 #pragma unroll
@@ -199,6 +204,14 @@ grouped_gemm_bf16_kernel(GroupedArgs g) {
         acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(fa[s], fw[s][j], acc[j], 0, 0, 0);
   }
 
+  if constexpr (PAIRED) {
+    if (wn & 1) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) up_sums[wn >> 1][lane][i] = acc[0][i];
+    }
+    __syncthreads();
+    if (wn & 1) return;
+  }
   TO* out = (TO*)g.out;
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
@@ -210,7 +223,9 @@ grouped_gemm_bf16_kernel(GroupedArgs g) {
     for (int j = 0; j < NB; ++j) {
       const int n = n0 + j * 16 + r16;
       if (n >= N) continue;
-      if constexpr (GATED)
+      if constexpr (PAIRED)
+        out[d * N + n] = from_f32<TO>(expert_unit(g, acc[j][i], up_sums[wn >> 1][lane][i], w));
+      else if constexpr (GATED)
         out[d * N + n] = from_f32<TO>(expert_unit(g, acc[2 * j][i], acc[2 * j + 1][i], w));
       else
         out[d * N + n] = from_f32<TO>(expert_act(acc[j][i], g.act) * g.out_scale * w);
@@ -441,7 +456,7 @@ extern "C" int za_grouped_gemm(const void* src, int src_dtype, long long src_row
     // a decode batch (an expert has a token or two): tiles of 16 rows
     const bool small = A <= 4LL * experts || A <= 64;
     const int TM = small ? 16 : 64;
-    const int columns = gate && !small ? 32 : 64;
+    const int columns = gate ? 32 : 64;
     dim3 grid((unsigned)((A + TM - 1) / TM + experts), (unsigned)((N + columns - 1) / columns)), block(256);
 #define ZA_GG(TMM, TO)                                                                          \
   {                                                                                             \
